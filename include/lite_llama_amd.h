@@ -607,12 +607,14 @@ int ll_qk_norm_cache(const void* qkv, int64_t ld, const void* q_w, const void* k
  * token_table[seq_req[tok_seq[t]]][pos]); score = (q . k) scale; sink [heads] or NULL adds exp(sink_h) to the denominator.
  * window > 0: only the last `window` positions (the token's own included) are seen, and besides them the sequence's first
  * keep_first positions.  k_stride / v_stride: elements between cache rows (>= kv_heads dk / kv_heads dv; the value rows may
- * be a column range of the key rows); out_stride: elements between output rows (>= heads dv). */
+ * be a column range of the key rows); out_stride: elements between output rows (>= heads dv).  cap > 0: scaled scores become
+ * cap tanh(score / cap); dist_bias (fp32 [heads][dist_n], or NULL): then dist_bias[h][min(tok_pos - key position, dist_n - 1)] is
+ * added. */
 int ll_ragged_attention(const void* q, const void* k_cache, const void* v_cache, const int32_t* token_table,
                         int64_t tt_stride, const int32_t* seq_req, const int32_t* tok_seq, const int32_t* tok_pos,
                         const void* sink, float scale, void* out, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk,
                         int64_t dv, int64_t k_stride, int64_t v_stride, int64_t window, int64_t keep_first,
-                        int64_t out_stride, int dtype, void* stream);
+                        int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, int dtype, void* stream);
 /* Rows [q (heads dk) | k (kv_heads dk) | v (kv_heads dv)] of stride ld, channel by channel in fp32: + bias [channels] (or NULL);
  * y_t = sum_j conv_w[c][j] u_(t - taps + 1 + j) over the sequence's positions (zeros in front of position 0; taps == 0: none),
  * the raw rows of a sequence's last taps - 1 positions carried in conv_state [2][state_half] (half seq_parity read, the other
@@ -643,7 +645,8 @@ int ll_ragged_attention_mfma(const void* q, const void* k_cache, const void* v_c
                              const int32_t* seq_first_pos, const void* sink, float scale, void* out, int64_t n,
                              int64_t batch, int64_t longest_run, int64_t longest_context, int decode, float* partials,
                              int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv, int64_t k_stride, int64_t v_stride,
-                             int64_t window, int64_t keep_first, int64_t out_stride, int dtype, void* stream);
+                             int64_t window, int64_t keep_first, int64_t out_stride, float cap, const float* dist_bias,
+                             int64_t dist_n, int dtype, void* stream);
 
 /* ---- sublayers between two grouped norms with a gated residual branch (csrc/group_norm.hip) --------------------------------
  * ll_gated_group_norm: with y: s = (sum of `parts` rows y[t][p][:] + shared_scale[t] * shared[t][:]) * sigmoid(gate[t][:] +
@@ -657,7 +660,8 @@ int ll_gated_group_norm(const float* x_in, float* x_out, void* h_out, const void
                         const void* post_w, const void* next_w, int64_t n, int64_t width, int64_t groups, float eps,
                         const void* y_bias, int dtype, void* stream);
 /* out [n, ff] (rows of stride out_ld) = act(gate[t][j]) * up[t][j], gate / up rows of stride gate_ld / up_ld; kind 0: silu,
- * 1: gelu (tanh form), 2: sigmoid, 3: clamped -- g = min(gate, p0), u = clamp(up, -p0, p0), g sigmoid(p1 g) (u + 1). */
+ * 1: gelu (tanh form), 2: sigmoid, 3: clamped -- g = min(gate, p0), u = clamp(up, -p0, p0), g sigmoid(p1 g) (u + 1); 4: relu(gate)^2,
+ * no up value enters (up may be NULL). */
 int ll_glu_act(void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const void* up, int64_t up_ld, int64_t n,
                int64_t ff, int kind, float p0, float p1, int dtype, void* stream);
 /* x <- cap * tanh(x / cap), in place. */
@@ -671,6 +675,16 @@ int64_t ll_mingru_scan_scratch_floats(int64_t batch, int64_t width, int64_t long
 int ll_mingru_scan(const void* z, const void* x, const void* g, int64_t ld, const void* z_bias, const void* x_bias,
                    void* out, int64_t batch, int64_t width, const int32_t* seq_start, const int32_t* seq_first_pos,
                    const int32_t* seq_slot, float* state, int64_t longest_run, float* scratch, int dtype, void* stream);
+/* RG-LRU: r = sigmoid(r_raw + r_bias), i = sigmoid(i_raw + i_bias), log a = -8 r softplus(lam), S <- a S + sqrt(1 - a^2) i u per
+ * channel, out = S * gelu(y) (tanh form).  The gate rows are those of a block-diagonal product over `blocks` equal parts of the
+ * channels: part p holds [r | i] at columns 2 p width / blocks ..  state [slots][width] fp32 (read when seq_first_pos > 0, written at
+ * the end of the run).  scratch (fp32, ll_rglru_scan_scratch_floats(...) floats, > 0 for runs of 128 tokens and more): long runs are
+ * walked in chunks side by side, as ll_mingru_scan's. */
+int64_t ll_rglru_scan_scratch_floats(int64_t n, int64_t batch, int64_t width, int64_t longest_run);
+int ll_rglru_scan(const void* u, int64_t u_ld, const void* gates, int64_t g_ld, const void* r_bias, const void* i_bias,
+                  const void* lam, const void* y, int64_t y_ld, void* out, int64_t n, int64_t batch, int64_t width,
+                  int64_t blocks, const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot,
+                  float* state, int64_t longest_run, float* scratch, int dtype, void* stream);
 
 /* ---- attention over a shared latent (csrc/latent_attn.hip) ------------------------------------------------------------------
  * ll_latent_kv_prep: rows (stride ld) hold the latent [rank] and the rotated key part [rot] at column kv_off: the cache row
@@ -695,12 +709,14 @@ int ll_rotate_pairs(const void* q, int64_t q_tok_stride, int64_t q_head_stride, 
  * are chosen and their weights are the softmax over the chosen logits alone (times route_scale).  scoring 2: scores =
  * softmax over all logits; ranked by score + correction[e] (storage dtype, or NULL); weights = the chosen scores themselves;
  * the last `identity` experts return the token's own row: their slots keep ids >= experts - identity (never placed by
- * ll_moe_sort over the experts that have weights) and extra_scale[t] receives the sum of their scores.
+ * ll_moe_sort over the experts that have weights) and extra_scale[t] receives the sum of their scores.  scoring 3: as 0, but the
+ * weights are the chosen sigmoid scores themselves.
  * ll_moe_sort: slots sorted by expert in blocks of `block` = ll_moe_rows_block(...) rows, 32 or 128 (counts: int32 scratch
  * [experts]; sorted [num_slots + experts (block - 1)], block_expert [ceil(that / block)], num_post [1]).
  * ll_moe_rows_gemm: glu != 0: w [experts][2 N][K] (gate rows, then up rows), out[slot] = silu(a Wg^T) * (a Wu^T) with
  * a = row slot / a_div (glu == 2: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit));
- * glu == 0: w [experts][N][K], out[slot] = (a W^T) * slot_weight[slot]. */
+ * glu == 0: w [experts][N][K], out[slot] = (a W^T) * slot_weight[slot]; glu == 3: w [experts][N][K],
+ * out[slot] = relu(slot_weight[slot] (a W^T))^2. */
 int ll_group_router(const void* h, int64_t h_ld, const void* w_router, const void* w_extra, int64_t n, int64_t width,
                     int64_t experts, int64_t top, int64_t group_count, int64_t group_keep, float route_scale, int scoring,
                     int32_t* ids, float* weights, float* extra_scale, float* logits, const void* correction, int64_t identity,
@@ -725,8 +741,8 @@ int ll_moe_rows_gemm(const void* a, int64_t a_ld, int64_t a_div, const void* w, 
  * ll_gated_out_norm: o fp32 [n, width] -> RMS norm over `parts` equal consecutive parts, times w[(channel) mod w_len] (NULL:
  * none), times act(gate) (gate_kind 0 none, 1 silu, 2 sigmoid; gate_first: before the norm), times out_scale -> out rows of
  * stride out_ld.
- * ll_conv_act: out = silu(bias + causal convolution over a sequence's positions of rows [n, >= channels] with w
- * [channels, taps]); state [2][slots][taps - 1][channels] (storage dtype; halves of state_half elements) carries the raw rows of
+ * ll_conv_act: out = bias + causal convolution (act != 0: silu of it) over a sequence's positions of rows [n, >= channels] with w
+ * [channels, taps]; state [2][slots][taps - 1][channels] (storage dtype; halves of state_half elements) carries the raw rows of
  * a sequence's last positions, double-buffered by seq_parity.
  * ll_rownorm_rope_cache: rows [q | k | v]; q and k RMS-normed over their whole row times q_w / k_w (NULL: no norm), entry i <
  * pairs of every head rotated with entry i + pairs by tok_pos * freq[i]; q -> q_out [n, heads, dk], k and value_scale * v ->
@@ -744,11 +760,37 @@ int ll_gated_out_norm(void* out, int64_t out_ld, const float* o, const void* gat
 int ll_conv_act(void* out, int64_t out_ld, const void* rows, int64_t ld, const void* w, const void* bias, int64_t channels,
                 int64_t taps, void* state, int64_t state_half, const int32_t* tok_seq, const int32_t* tok_pos,
                 const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, const int32_t* seq_parity,
-                int64_t n, int dtype, void* stream);
+                int64_t n, int act, int dtype, void* stream);
 int ll_rownorm_rope_cache(const void* rows, int64_t ld, const void* q_w, const void* k_w, float eps, const float* freq,
                           int64_t pairs, float value_scale, const int32_t* tok_pos, const int32_t* select, void* q_out,
                           void* k_cache, void* v_cache, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv,
                           int dtype, void* stream);
+
+/* ---- gated delta rule (csrc/delta_scan.hip) -----------------------------------------------------------------------------------
+ * Per head, fp32 state [slots, heads, dk, dv]: S <- diag(g) S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q.  Rows k / q hold one
+ * raw key / query head per heads / qk_rep value heads; a head is divided by sqrt(sum of squares + unit_eps), q also times q_scale.
+ * g = exp(-exp(a_log[h]) softplus(gate[t][h dk + i] + dt_bias[h dk + i])) per key entry, beta = sigmoid(beta[t][h]).  o: fp32
+ * [n, heads dv].  A run that starts at position 0 starts from zeros.  scratch (fp32, 16-byte aligned, ll_delta_scan_scratch_floats
+ * floats, or NULL): decays and per-token scalars are evaluated once, ahead of the walk (same values).  longest_run: most tokens a
+ * sequence of the step brings (0: unknown); sizes the staging buffers only.  dk <= 256. */
+int ll_delta_scan_supported(int64_t dk, int64_t dv);
+int64_t ll_delta_scan_scratch_floats(int64_t n, int64_t heads, int64_t dk);
+int ll_delta_scan(const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, int64_t heads,
+                  int64_t dk, int64_t dv, int64_t qk_rep, float q_scale, float unit_eps, const void* gate, int64_t gate_ld,
+                  const void* dt_bias, const void* a_log, const void* beta, int64_t beta_ld, float* o, int64_t batch,
+                  const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, float* state,
+                  float* scratch, int64_t n, int64_t longest_run, int dtype, void* stream);
+
+/* ---- several mixed residual streams (csrc/stream_norm.hip) --------------------------------------------------------------------
+ * With y: d = (sum of `parts` rows y[t][p][:] + shared_scale[t] * shared[t][:]) * scale (shared, scale may be NULL) and
+ * x_out[t][to] = sum_s mix[s][to] x_in[t][s] + out_w[to] d for all `streams` rows of width elements; without y x_in is only read.
+ * When h is given: u = sum_s in_w[s] x[t][s] of the new streams (in_w NULL: ones), h = u / sqrt(mean(u^2) + eps) * (weight_base +
+ * norm_w).  x_in: token stride in_tok, stream stride in_stream (0: one row that every stream reads); x_out [n][streams][width] may
+ * be x_in when that has the same layout.  streams <= 32. */
+int ll_stream_norm(const float* x_in, int64_t in_tok, int64_t in_stream, float* x_out, const void* y, int64_t parts,
+                   const void* shared, const float* shared_scale, const void* scale, const void* mix, const void* out_w,
+                   const void* in_w, const void* norm_w, float weight_base, float eps, void* h, int64_t n, int64_t width,
+                   int64_t streams, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

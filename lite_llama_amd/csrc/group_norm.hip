@@ -11,6 +11,7 @@
 //                         the next sublayer (or the output head).  Without a pending result it is the plain grouped norm.
 //   ll_glu_act            act(gate) * up, gate and up two row-strided column ranges (act: silu, the tanh form of gelu, sigmoid),
 //                         or the clamped form g sigmoid(a g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit);
+//                         or, without an up range, the square of relu;
 //                         the result may be a column range of wider rows
 //
 // Storage dtype DT = LL_F16 / LL_BF16 / LL_F32 for activations and weights; sums, norms, gates and the residual are fp32.
@@ -279,7 +280,8 @@ template <int DT>
 __device__ __forceinline__ float glu_value(float g, float u, int kind);
 
 // out[t][j] = act(gate[t][j]) * up[t][j]; gate and up rows have their own strides (two column ranges of one projection, or two
-// tensors).  kind 0: silu, 1: gelu (tanh form), 2: sigmoid, 3: clamped (p0 = limit, p1 = slope inside the sigmoid)
+// tensors).  kind 0: silu, 1: gelu (tanh form), 2: sigmoid, 3: clamped (p0 = limit, p1 = slope inside the sigmoid), 4: relu(gate)^2
+// (no up value enters)
 template <int DT>
 __device__ __forceinline__ float glu_value(float g, float u, int kind, float p0, float p1) {
   constexpr bool EXACT = DT == LL_F32;
@@ -292,6 +294,9 @@ __device__ __forceinline__ float glu_value(float g, float u, int kind, float p0,
     g = fminf(g, p0);
     u = fminf(fmaxf(u, -p0), p0) + 1.0f;
     a = g * sigmoid_f<EXACT>(p1 * g);
+  } else if (kind == 4) {
+    g = fmaxf(g, 0.f);
+    return g * g;
   } else {
     const float inner = 0.7978845608028654f * (g + 0.044715f * g * g * g);
     const float th = EXACT ? tanhf(inner) : 2.0f * ll_sigmoidf(2.0f * inner) - 1.0f;
@@ -397,8 +402,12 @@ extern "C" int ll_gated_group_norm(const float* x_in, float* x_out, void* h_out,
 extern "C" int ll_glu_act(void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const void* up, int64_t up_ld, int64_t n,
                           int64_t ff, int kind, float p0, float p1, int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
-  if (n < 0 || ff < 1 || out_ld < ff || gate_ld < ff || up_ld < ff || ff > (1 << 24) || kind < 0 || kind > 3) return LL_ERR_SHAPE;
+  if (n < 0 || ff < 1 || out_ld < ff || gate_ld < ff || (kind != 4 && up_ld < ff) || ff > (1 << 24) || kind < 0 || kind > 4) return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
+  if (kind == 4) {   // (one input range: it is passed on as both)
+    up = gate;
+    up_ld = gate_ld;
+  }
   if (!out || !gate || !up) return LL_ERR_ARG;
   hipStream_t st = (hipStream_t)stream;
   const int vec = dtype == LL_F32 ? 4 : 8;

@@ -11,7 +11,7 @@
 //   ll_gated_out_norm       o (fp32) -> RMS norm over equal consecutive parts of the row, times a weight (one per channel, or a
 //                           shorter vector repeated), times silu / sigmoid of a gate row -- before or after the norm --, times a
 //                           constant -> storage dtype, into a column range of the next projection's input
-//   ll_conv_act             causal convolution over time per channel (+ bias) and silu, the raw rows of a sequence's last
+//   ll_conv_act             causal convolution over time per channel (+ bias), with or without silu, the raw rows of a sequence's last
 //                           taps - 1 positions carried per sequence slot
 //   ll_rownorm_rope_cache   [q | k | v] rows -> q and k RMS-normed over their WHOLE row (all heads at once, a weight per entry),
 //                           entry i of a head's first `dims` entries rotated with entry i + dims / 2 by position * f_i; k and
@@ -226,8 +226,8 @@ __global__ __launch_bounds__(256) void gated_out_norm_kernel(void* __restrict__ 
   }
 }
 
-// Thread per (token, channel): y = silu(bias + sum_j w[c][j] u_(p - taps + 1 + j)), positions in front of the sequence count
-// as zero.  A predecessor that rides in the same step is read from the step's rows, an earlier one from the carried rows
+// Thread per (token, channel): y = act(bias + sum_j w[c][j] u_(p - taps + 1 + j)), act = silu or nothing, positions in front of the
+// sequence count as zero.  A predecessor that rides in the same step is read from the step's rows, an earlier one from the carried rows
 // (state [2][slots][taps - 1][channels]: the half named by the sequence's parity is read, the other written by the run's last
 // token from the same two sources, so runs shorter than the taps shift the old rows forward).
 template <int DT>
@@ -236,7 +236,7 @@ __global__ __launch_bounds__(256) void conv_act_kernel(void* __restrict__ out, i
                                                        void* __restrict__ state, int64_t state_half, const int32_t* __restrict__ tok_seq,
                                                        const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ seq_start,
                                                        const int32_t* __restrict__ seq_first_pos, const int32_t* __restrict__ seq_slot,
-                                                       const int32_t* __restrict__ seq_parity) {
+                                                       const int32_t* __restrict__ seq_parity, int act) {
   const int64_t t = blockIdx.x;
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= channels) return;
@@ -255,7 +255,7 @@ __global__ __launch_bounds__(256) void conv_act_kernel(void* __restrict__ out, i
     if (p < 0) continue;
     acc += ldv<DT>(w, (int64_t)c * taps + j) * raw_at(p);
   }
-  stv<DT>(out, t * out_ld + c, acc * act_sigmoid<DT>(acc));
+  stv<DT>(out, t * out_ld + c, act ? acc * act_sigmoid<DT>(acc) : acc);
   if (taps > 1 && t == seq_start[seq + 1] - 1) {
     for (int s = 0; s < taps - 1; ++s) {
       const int p = pos + 1 - (taps - 1) + s;
@@ -383,7 +383,7 @@ __global__ __launch_bounds__(256) void conv_act_vec_kernel(void* __restrict__ ou
                                                            void* __restrict__ state, int64_t state_half, const int32_t* __restrict__ tok_seq,
                                                            const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ seq_start,
                                                            const int32_t* __restrict__ seq_first_pos, const int32_t* __restrict__ seq_slot,
-                                                           const int32_t* __restrict__ seq_parity, int64_t pieces) {
+                                                           const int32_t* __restrict__ seq_parity, int64_t pieces, int act) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= pieces) return;
   const int per = channels >> 3;
@@ -421,8 +421,10 @@ __global__ __launch_bounds__(256) void conv_act_vec_kernel(void* __restrict__ ou
 #pragma unroll
     for (int e = 0; e < 8; ++e) acc[e] += wl[e * TAPS + j] * u[e];
   }
+  if (act) {
 #pragma unroll
-  for (int e = 0; e < 8; ++e) acc[e] = acc[e] * act_sigmoid<DT>(acc[e]);
+    for (int e = 0; e < 8; ++e) acc[e] = acc[e] * act_sigmoid<DT>(acc[e]);
+  }
   st8<DT>(out, t * out_ld + c, acc);
   if (TAPS > 1 && t == seq_start[seq + 1] - 1) {
 #pragma unroll
@@ -608,7 +610,7 @@ extern "C" int ll_gated_out_norm(void* out, int64_t out_ld, const float* o, cons
 extern "C" int ll_conv_act(void* out, int64_t out_ld, const void* rows, int64_t ld, const void* w, const void* bias, int64_t channels,
                            int64_t taps, void* state, int64_t state_half, const int32_t* tok_seq, const int32_t* tok_pos,
                            const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, const int32_t* seq_parity,
-                           int64_t n, int dtype, void* stream) {
+                           int64_t n, int act, int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
   if (n < 0 || channels < 1 || taps < 1 || taps > 64 || ld < channels || out_ld < channels || (channels + 255) / 256 > 65535)
     return LL_ERR_SHAPE;
@@ -623,7 +625,7 @@ extern "C" int ll_conv_act(void* out, int64_t out_ld, const void* rows, int64_t 
     const dim3 vgrid((unsigned)((pieces + 255) / 256));
 #define CALL_T(DT, T)                                                                                                                \
   conv_act_vec_kernel<DT, T><<<vgrid, 256, 0, (hipStream_t)stream>>>(out, out_ld, rows, ld, w, bias, (int)channels, state, state_half, \
-                                                                     tok_seq, tok_pos, seq_start, seq_first_pos, seq_slot, seq_parity, pieces)
+                                                                     tok_seq, tok_pos, seq_start, seq_first_pos, seq_slot, seq_parity, pieces, act)
 #define CALL(DT)                      \
   if (taps == 1) CALL_T(DT, 1);       \
   else if (taps == 2) CALL_T(DT, 2);  \
@@ -637,7 +639,7 @@ extern "C" int ll_conv_act(void* out, int64_t out_ld, const void* rows, int64_t 
   const dim3 grid((unsigned)n, (unsigned)((channels + 255) / 256));
 #define CALL(DT)                                                                                                                     \
   conv_act_kernel<DT><<<grid, 256, 0, (hipStream_t)stream>>>(out, out_ld, rows, ld, w, bias, (int)channels, (int)taps, state, state_half, \
-                                                             tok_seq, tok_pos, seq_start, seq_first_pos, seq_slot, seq_parity)
+                                                             tok_seq, tok_pos, seq_start, seq_first_pos, seq_slot, seq_parity, act)
   LL_BY_DTYPE(dtype, CALL);
 #undef CALL
   return LL_LAUNCH_CHECK();

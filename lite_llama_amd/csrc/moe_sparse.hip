@@ -9,8 +9,9 @@
 //                     that selects by ranks (ties: the lower index first), so slot k of a token holds its k-th best expert.
 //   ll_moe_sort       slots (token, k) sorted by expert, every expert's run padded to the row-block size with a sentinel:
 //                     sorted_ids / block_expert / num_post as in moe_align_block_size.  Deterministic: no atomics.
-//   ll_moe_rows_gemm  the grouped products over sorted row blocks: either act = silu(a Wg_e^T) * (a Wu_e^T) (gate and up rows
-//                     stacked in one matrix per expert) or out = (a W_e^T) * slot weight, fp32 accumulation.  MFMA form for
+//   ll_moe_rows_gemm  the grouped products over sorted row blocks: act = silu(a Wg_e^T) * (a Wu_e^T) (gate and up rows
+//                     stacked in one matrix per expert), out = (a W_e^T) * slot weight, or act = relu((slot weight * a) W_e^T)^2 (experts
+//                     without a gate whose weight multiplies their INPUT), fp32 accumulation.  MFMA form for
 //                     16-bit storage with contraction widths that are multiples of 8, a plain tiled form otherwise.
 #include "common.h"
 
@@ -30,6 +31,18 @@ __device__ __forceinline__ void stv(void* p, int64_t i, float v) {
 }
 
 __device__ __forceinline__ float sigmoid_exact(float v) { return 1.0f / (1.0f + expf(-v)); }
+
+// what one row block of the grouped products does with its sums: 0 times the slot's weight, 1 a gated pair (glu_pair), 2 the square
+// of relu of the sum times the slot's weight (the weight multiplies the expert's input: the sum is linear in it)
+template <int MODE>
+__device__ __forceinline__ float slot_value(float sum, float weight) {
+  const float v = sum * weight;
+  if constexpr (MODE == 2) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+  }
+  return v;
+}
 
 // the gated pair of an expert's first product.  limit < 0: silu(g) u; else the clamped form g' sigmoid(1.702 g') (u' + 1) with
 // g' = min(g, limit), u' = clamp(u, -limit, limit)
@@ -118,7 +131,8 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const void* __restri
 // groups) and the weights are the softmax over the chosen logits alone; 2: scores = softmax over ALL logits (no groups), the
 // experts are ranked by score + correction[e], the weights are the chosen scores themselves (not renormalised); the last
 // `identity` experts have no weights of their own -- a slot that chose one keeps its id (>= experts - identity, which the sort
-// by expert never places) and its score is added to extra_scale[t], the factor of the token's own input row
+// by expert never places) and its score is added to extra_scale[t], the factor of the token's own input row; 3: sigmoid scores
+// as in 0, but the weights are the chosen scores themselves (not renormalised)
 template <int SCORING, int DT = LL_F32>
 __global__ __launch_bounds__(64) void group_select_kernel(const float* __restrict__ logits, int rows, int experts, int top,
                                                           int group_count, int group_keep, float route_scale,
@@ -213,6 +227,8 @@ __global__ __launch_bounds__(64) void group_select_kernel(const float* __restric
   if constexpr (SCORING == 1) {   // chosen[0] is the largest: exp(z - z_max) summed in slot order by every lane
     for (int k = 0; k < top; ++k) sum += expf(chosen[k] - chosen[0]);
     for (int k = lane; k < top; k += 64) weights[t * top + k] = expf(chosen[k] - chosen[0]) / sum * route_scale;
+  } else if constexpr (SCORING == 3) {
+    for (int k = lane; k < top; k += 64) weights[t * top + k] = chosen[k] * route_scale;
   } else {
     for (int k = 0; k < top; ++k) sum += chosen[k];
     for (int k = lane; k < top; k += 64) weights[t * top + k] = chosen[k] / (sum + 1e-20f) * route_scale;
@@ -264,13 +280,14 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const int32_t* __restric
 // ------------------------------------------------------------------------------------------------------------------------
 // grouped products, plain tiled form: 32 sorted rows x 64 columns per workgroup, 32 contraction entries per pass
 // ------------------------------------------------------------------------------------------------------------------------
-template <int DT, bool GLU>
+template <int DT, int MODE>
 __global__ __launch_bounds__(256) void moe_rows_gemm_kernel(const void* __restrict__ a, int64_t a_ld, int a_div,
                                                             const void* __restrict__ w, int64_t w_stride_e, int K, int N,
                                                             const float* __restrict__ slot_weight, void* __restrict__ out,
                                                             int64_t out_ld, const int32_t* __restrict__ sorted,
                                                             const int32_t* __restrict__ block_expert,
                                                             const int32_t* __restrict__ num_post, int num_slots, float glu_limit) {
+  constexpr bool GLU = MODE == 1;
   constexpr int BM = 32, BN = 64, BK = 32;
   __shared__ float As[BM][BK + 1];
   __shared__ int rows[BM];
@@ -318,7 +335,7 @@ __global__ __launch_bounds__(256) void moe_rows_gemm_kernel(const void* __restri
     if (GLU) {
       v = glu_pair<DT>(acc_g[r], acc_u[r], glu_limit);
     } else {
-      v = slot_weight ? acc_g[r] * slot_weight[slot] : acc_g[r];
+      v = slot_value<MODE>(acc_g[r], slot_weight ? slot_weight[slot] : 1.0f);
     }
     stv<DT>(out, (int64_t)slot * out_ld + col, v);
   }
@@ -341,13 +358,14 @@ __device__ __forceinline__ f32x4 mfma16(const Q4& a, const Q4& b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-template <int DT, bool GLU>
+template <int DT, int MODE>
 __global__ __launch_bounds__(64) void moe_rows_gemm_mfma_kernel(const uint16_t* __restrict__ a, int64_t a_ld, int a_div,
                                                                 const uint16_t* __restrict__ w, int64_t w_stride_e, int K, int N,
                                                                 const float* __restrict__ slot_weight, uint16_t* __restrict__ out,
                                                                 int64_t out_ld, const int32_t* __restrict__ sorted,
                                                                 const int32_t* __restrict__ block_expert,
                                                                 const int32_t* __restrict__ num_post, int num_slots, float glu_limit) {
+  constexpr bool GLU = MODE == 1;
   constexpr int BM = 32, BN = 32;
   constexpr int NW = GLU ? 4 : 2;   // weight-row tiles of 16: gate 0..1, up 2..3
   const int block = blockIdx.x;
@@ -413,7 +431,7 @@ __global__ __launch_bounds__(64) void moe_rows_gemm_mfma_kernel(const uint16_t* 
           const float g = acc[j][m][r];
           v = glu_pair<DT>(g, acc[j + 2][m][r], glu_limit);
         } else {
-          v = acc[j][m][r] * sw;
+          v = slot_value<MODE>(acc[j][m][r], sw);
         }
         orow[col] = from_f32<DT>(v);
       }
@@ -428,13 +446,14 @@ __global__ __launch_bounds__(64) void moe_rows_gemm_mfma_kernel(const uint16_t* 
 // products); a wave multiplies all eight row tiles with two weight tiles (its gate and its up tile), so every A fragment read
 // from LDS feeds two MFMAs and every weight fragment eight.
 // ------------------------------------------------------------------------------------------------------------------------
-template <int DT, bool GLU>
+template <int DT, int MODE>
 __global__ __launch_bounds__(256) void moe_rows_gemm_tiled_kernel(const uint16_t* __restrict__ a, int64_t a_ld, int a_div,
                                                                   const uint16_t* __restrict__ w, int64_t w_stride_e, int K, int N,
                                                                   const float* __restrict__ slot_weight, uint16_t* __restrict__ out,
                                                                   int64_t out_ld, const int32_t* __restrict__ sorted,
                                                                   const int32_t* __restrict__ block_expert,
                                                                   const int32_t* __restrict__ num_post, int num_slots, float glu_limit) {
+  constexpr bool GLU = MODE == 1;
   constexpr int BM = 128, WN = 128, BK = 64, STR = BK + 8, CW = GLU ? 64 : 128;
   __shared__ __attribute__((aligned(16))) uint16_t lds_a[BM * STR];
   __shared__ __attribute__((aligned(16))) uint16_t lds_w[WN * STR];
@@ -515,7 +534,7 @@ __global__ __launch_bounds__(256) void moe_rows_gemm_tiled_kernel(const uint16_t
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int col = n0 + 16 * (2 * wave + j) + 4 * c + r;
-          if (col < N) orow[col] = from_f32<DT>(acc[j][m][r] * sw);
+          if (col < N) orow[col] = from_f32<DT>(slot_value<MODE>(acc[j][m][r], sw));
         }
     }
   }
@@ -541,7 +560,7 @@ extern "C" int ll_group_router(const void* h, int64_t h_ld, const void* w_router
   if (scoring != 2 && (correction || identity)) return LL_ERR_SHAPE;
   if (n < 0 || width < 1 || h_ld < width || experts < 1 || experts > 4096 || top < 1 || top > experts || top > 64 || group_count < 1 ||
       experts % group_count || group_keep < 1 || group_keep > group_count || group_keep * (experts / group_count) < top ||
-      scoring < 0 || scoring > 2 || (scoring == 1 && group_count != 1))
+      scoring < 0 || scoring > 3 || (scoring == 1 && group_count != 1))
     return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
   if (!h || !w_router || !ids || !weights || !logits || (w_extra && !extra_scale)) return LL_ERR_ARG;
@@ -578,6 +597,9 @@ extern "C" int ll_group_router(const void* h, int64_t h_ld, const void* w_router
   } else if (scoring == 1)
     group_select_kernel<1><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,
                                                                route_scale, ids, weights, extra_scale);
+  else if (scoring == 3)
+    group_select_kernel<3><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,
+                                                               route_scale, ids, weights, extra_scale);
   else
     group_select_kernel<0><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,
                                                                route_scale, ids, weights, extra_scale);
@@ -606,14 +628,17 @@ extern "C" int ll_moe_sort(const int32_t* ids, int64_t num_slots, int64_t expert
 
 // glu != 0: w [experts][2 N][K] (gate rows, then up rows), out[slot][N] = silu(a_row Wg^T) * (a_row Wu^T) with a_row =
 // a[slot / a_div] (glu == 2: the clamped pair g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = clamp(u, +-limit)); glu == 0: w [experts][N][K], out[slot][N] = (a[slot / a_div] W^T) * slot_weight[slot] (NULL: 1).
+// glu == 3: w [experts][N][K], out[slot][N] = relu(slot_weight[slot] (a[slot / a_div] W^T))^2: an expert without a gate whose weight
+// multiplies its input.
 extern "C" int ll_moe_rows_gemm(const void* a, int64_t a_ld, int64_t a_div, const void* w, int64_t w_stride_e, int64_t K, int64_t N,
                                 int glu, const float* slot_weight, void* out, int64_t out_ld, const int32_t* sorted,
                                 const int32_t* block_expert, const int32_t* num_post, int64_t num_slots, int64_t experts,
                                 int64_t block, float limit, int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
-  if (glu < 0 || glu > 2 || (glu == 2 && !(limit >= 0.f))) return LL_ERR_SHAPE;
+  if (glu < 0 || glu > 3 || (glu == 2 && !(limit >= 0.f))) return LL_ERR_SHAPE;
+  const int mode = glu == 3 ? 2 : glu ? 1 : 0;   // (which epilogue; 1: gate and up rows)
   const float glu_limit = glu == 2 ? limit : -1.0f;
-  if (num_slots < 0 || K < 1 || N < 1 || a_div < 1 || a_ld < K || out_ld < N || w_stride_e < (glu ? 2 : 1) * N * K || experts < 1 ||
+  if (num_slots < 0 || K < 1 || N < 1 || a_div < 1 || a_ld < K || out_ld < N || w_stride_e < (mode == 1 ? 2 : 1) * N * K || experts < 1 ||
       (block != 32 && block != 128))
     return LL_ERR_SHAPE;
   if (num_slots == 0) return LL_OK;
@@ -624,13 +649,13 @@ extern "C" int ll_moe_rows_gemm(const void* a, int64_t a_ld, int64_t a_div, cons
   const bool mfma = !no_mfma && dtype != LL_F32 && K % 8 == 0 && a_ld % 8 == 0 && w_stride_e % 8 == 0 && ll_aligned16(a) && ll_aligned16(w);
   if (block == 128) {
     if (!mfma) return LL_ERR_SHAPE;   // (blocks of 128 rows are only sorted for the tiled matrix-core form)
-    const dim3 grid((unsigned)max_blocks, (unsigned)((N + (glu ? 63 : 127)) / (glu ? 64 : 128)));
+    const dim3 grid((unsigned)max_blocks, (unsigned)((N + (mode == 1 ? 63 : 127)) / (mode == 1 ? 64 : 128)));
 #define CALL_T(DT, G)                                                                                                          \
   moe_rows_gemm_tiled_kernel<DT, G><<<grid, 256, 0, st>>>((const uint16_t*)a, a_ld, (int)a_div, (const uint16_t*)w, w_stride_e, \
                                                           (int)K, (int)N, slot_weight, (uint16_t*)out, out_ld, sorted, block_expert, \
                                                           num_post, (int)num_slots, glu_limit)
-    if (dtype == LL_F16) { if (glu) CALL_T(LL_F16, true); else CALL_T(LL_F16, false); }
-    else { if (glu) CALL_T(LL_BF16, true); else CALL_T(LL_BF16, false); }
+    if (dtype == LL_F16) { if (mode == 1) CALL_T(LL_F16, 1); else if (mode == 2) CALL_T(LL_F16, 2); else CALL_T(LL_F16, 0); }
+    else { if (mode == 1) CALL_T(LL_BF16, 1); else if (mode == 2) CALL_T(LL_BF16, 2); else CALL_T(LL_BF16, 0); }
 #undef CALL_T
     return LL_LAUNCH_CHECK();
   }
@@ -640,18 +665,21 @@ extern "C" int ll_moe_rows_gemm(const void* a, int64_t a_ld, int64_t a_div, cons
   moe_rows_gemm_mfma_kernel<DT, G><<<grid, 64, 0, st>>>((const uint16_t*)a, a_ld, (int)a_div, (const uint16_t*)w, w_stride_e, \
                                                         (int)K, (int)N, slot_weight, (uint16_t*)out, out_ld, sorted, block_expert, \
                                                         num_post, (int)num_slots, glu_limit)
-    if (dtype == LL_F16) { if (glu) CALL_M(LL_F16, true); else CALL_M(LL_F16, false); }
-    else { if (glu) CALL_M(LL_BF16, true); else CALL_M(LL_BF16, false); }
+    if (dtype == LL_F16) { if (mode == 1) CALL_M(LL_F16, 1); else if (mode == 2) CALL_M(LL_F16, 2); else CALL_M(LL_F16, 0); }
+    else { if (mode == 1) CALL_M(LL_BF16, 1); else if (mode == 2) CALL_M(LL_BF16, 2); else CALL_M(LL_BF16, 0); }
 #undef CALL_M
     return LL_LAUNCH_CHECK();
   }
   const dim3 grid((unsigned)max_blocks, (unsigned)((N + 63) / 64));
-#define CALL(DT)                                                                                                             \
-  if (glu) moe_rows_gemm_kernel<DT, true><<<grid, 256, 0, st>>>(a, a_ld, (int)a_div, w, w_stride_e, (int)K, (int)N, slot_weight, \
-                                                                out, out_ld, sorted, block_expert, num_post, (int)num_slots, glu_limit);    \
-  else moe_rows_gemm_kernel<DT, false><<<grid, 256, 0, st>>>(a, a_ld, (int)a_div, w, w_stride_e, (int)K, (int)N, slot_weight,   \
-                                                             out, out_ld, sorted, block_expert, num_post, (int)num_slots, glu_limit)
+#define CALL_P(DT, G)                                                                                                        \
+  moe_rows_gemm_kernel<DT, G><<<grid, 256, 0, st>>>(a, a_ld, (int)a_div, w, w_stride_e, (int)K, (int)N, slot_weight, out, out_ld, sorted, \
+                                                    block_expert, num_post, (int)num_slots, glu_limit)
+#define CALL(DT)                        \
+  if (mode == 1) CALL_P(DT, 1);         \
+  else if (mode == 2) CALL_P(DT, 2);    \
+  else CALL_P(DT, 0)
   LL_BY_DTYPE(dtype, CALL);
 #undef CALL
+#undef CALL_P
   return LL_LAUNCH_CHECK();
 }

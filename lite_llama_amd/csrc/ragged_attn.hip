@@ -12,7 +12,8 @@
 //                        layers and heads that rotate alike
 //   ll_ragged_attention  every token of the step against keys 0 .. its own position of its sequence, read through the
 //                        per-token row table; scores, softmax and the running output in fp32; optionally only the last
-//                        `window` keys plus the sequence's first `keep_first`
+//                        `window` keys plus the sequence's first `keep_first`; optionally scores capped to cap tanh(s / cap)
+//                        and a bias per head and distance added
 //
 // The sink is a virtual key with score sink_h (not scaled) and a zero value: the running softmax simply STARTS at
 // (max = sink, sum = 1, output = 0).  A token's result depends only on its own position and on the cache rows of its
@@ -484,7 +485,7 @@ __global__ __launch_bounds__(256) void ragged_attention_kernel(
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos, const void* __restrict__ sink, float scale,
     void* __restrict__ out, int64_t n, int heads, int kv_heads, int dk, int dv, int64_t k_stride, int64_t v_stride, int window,
-    int keep_first, int64_t out_stride) {
+    int keep_first, int64_t out_stride, float cap, const float* __restrict__ dist_bias, int dist_n) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   float* sq = lds + wave * (dk + 128);  // [dk] query
@@ -521,6 +522,8 @@ __global__ __launch_bounds__(256) void ragged_attention_kernel(
       row = table[j];
       const int64_t kb = (int64_t)row * k_stride + (int64_t)g * dk;
       s = dot_row<DT>(sq, k_cache, kb, dk, vec) * scale;
+      if (cap > 0.f) s = cap * tanhf(s / cap);
+      if (dist_bias) s += dist_bias[(int64_t)h * dist_n + (pos - j < dist_n ? pos - j : dist_n - 1)];
     }
     const float tile_max = wave_max(s);
     const float m_new = fmaxf(m, tile_max);
@@ -687,11 +690,11 @@ extern "C" int ll_ragged_attention(const void* q, const void* k_cache, const voi
                                    int64_t tt_stride, const int32_t* seq_req, const int32_t* tok_seq, const int32_t* tok_pos,
                                    const void* sink, float scale, void* out, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk,
                                    int64_t dv, int64_t k_stride, int64_t v_stride, int64_t window, int64_t keep_first,
-                                   int64_t out_stride, int dtype, void* stream) {
+                                   int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
   if (n < 0 || heads < 1 || kv_heads < 1 || heads % kv_heads || dk < 1 || dk > 1024 || dv < 1 || dv > 1024 || window < 0 ||
       window > 0x7fffffff || keep_first < 0 || keep_first > 0x7fffffff || k_stride < kv_heads * dk || v_stride < kv_heads * dv ||
-      out_stride < heads * dv)
+      out_stride < heads * dv || !(cap >= 0.f) || (dist_bias && (dist_n < 1 || dist_n > 0x7fffffff)))
     return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
   if (!q || !k_cache || !v_cache || !token_table || !seq_req || !tok_seq || !tok_pos || !out) return LL_ERR_ARG;
@@ -703,7 +706,7 @@ extern "C" int ll_ragged_attention(const void* q, const void* k_cache, const voi
 #define CALL_V(DT, V)                                                                                                        \
   ragged_attention_kernel<DT, V><<<grid, 256, lds, st>>>(q, k_cache, v_cache, token_table, tt_stride, seq_req, tok_seq, tok_pos, \
                                                          sink, scale, out, n, (int)heads, (int)kv_heads, (int)dk, (int)dv, k_stride, \
-                                                         v_stride, (int)window, (int)keep_first, out_stride)
+                                                         v_stride, (int)window, (int)keep_first, out_stride, cap, dist_bias, (int)dist_n)
 #define CALL(DT)                     \
   if (vpl == 1) CALL_V(DT, 1);       \
   else if (vpl == 2) CALL_V(DT, 2);  \

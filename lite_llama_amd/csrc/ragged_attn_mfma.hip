@@ -12,6 +12,8 @@
 // second product the fp32 weight is split into two 16-bit parts (p = hi + lo, two MFMAs) so that it enters with ~16 mantissa
 // bits instead of 8.  The sink starts the running softmax (max = sink, sum = 1) of a sequence's FIRST partition.
 // Widths that are not multiples of 32 (keys) / 16 (values) are zero-padded; both must be multiples of 8.
+// BIASED forms: scores capped to cap tanh(s / cap), then a bias per head and distance (dist_bias [heads][dist_n], fp32; distances
+// beyond the table read its last entry) is added; the softmax runs in base 2, so both enter times log2(e).
 #include "common.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -42,14 +44,31 @@ __device__ __forceinline__ void split2(float p, uint16_t& hi, uint16_t& lo) {
   else lo = from_f32<DT>(rest);
 }
 
+// what the BIASED forms do to a score: cap (0: none) and the bias table [heads][dist_n] (NULL: none)
+struct ScoreShape {
+  float scale, cap;
+  const float* dist_bias;
+  int dist_n;
+};
+
+// scaled dot product -> capped, biased score times log2(e); tanh(x) = 1 - 2 / (1 + e^(2x)) through the hardware exp2 / reciprocal
+__device__ __forceinline__ float shaped_score(float dot, const ScoreShape& sh, float bias) {
+  float s = dot * sh.scale;
+  if (sh.cap > 0.f) {
+    const float x = s * (1.0f / sh.cap);
+    s = sh.cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * (2.0f * kLog2e))));
+  }
+  return (s + bias) * kLog2e;
+}
+
 // Decoded tokens.  grid = (partitions of the longest context, kv_heads * column tiles per group, sequences)
-template <int DT, int NSM, int NTM>
+template <int DT, int NSM, int NTM, bool BIASED>
 __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ seq_start, const int32_t* __restrict__ seq_first_pos, const uint16_t* __restrict__ sink,
     float scale_log2, uint16_t* __restrict__ out, float* __restrict__ partials, int max_parts, int heads, int kv_heads, int dk,
-    int dv, int64_t k_stride, int64_t v_stride, int window, int shared_kv, int keep_first, int64_t out_stride) {
+    int dv, int64_t k_stride, int64_t v_stride, int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape) {
   static_assert(NTM / 2 == NSM, "value fragments of shared rows are the key fragments");
   constexpr int QB = 1;
   constexpr bool DECODE = true;
@@ -119,6 +138,15 @@ __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
     for (int i = 0; i < NTM; ++i) ot[qb][i] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
+  const float* bias_row = nullptr;   // this column's head in the bias table, and its entry for all far distances
+  float bias_far = 0.f;
+  if constexpr (BIASED) {
+    if (shape.dist_bias) {
+      bias_row = shape.dist_bias + (int64_t)head[0] * shape.dist_n;
+      bias_far = bias_row[shape.dist_n - 1];
+    }
+  }
+
   // K / V fragments of a tile are requested one tile ahead (and its cache rows two tiles ahead): the loads of tile i + 1 are in
   // flight under the products and the softmax of tile i
   #define zero4 (Q4{0, 0, 0, 0})
@@ -175,13 +203,28 @@ __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
       for (int s = 0; s < NSM; ++s)
         if (s < ns) sb = mfma16<DT>(kb[s], qf[qb][s], sb);
       // rows = keys p0 + 4 c + r (+ 16), column = query t
+      if constexpr (BIASED) {
+        const bool far = qpos[qb] - (p0 + 31) >= shape.dist_n - 1;   // (wave-uniform: one token) every key of the tile reads the last entry
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int da = qpos[qb] - (p0 + 4 * c + r), db = da - 16;   // distances; negative past the token (masked below)
+          float ba = bias_far, bb = bias_far;
+          if (!far && bias_row) {
+            ba = bias_row[da < 0 ? 0 : da < shape.dist_n ? da : shape.dist_n - 1];
+            bb = bias_row[db < 0 ? 0 : db < shape.dist_n ? db : shape.dist_n - 1];
+          }
+          sa[r] = shaped_score(sa[r], shape, ba);
+          sb[r] = shaped_score(sb[r], shape, bb);
+        }
+      }
+      const float mul = BIASED ? 1.0f : scale_log2;
       float sc[8];
       float mx = -INFINITY;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int k0i = p0 + 4 * c + r, k1i = k0i + 16;
-        sc[r] = (k0i <= qpos[qb] && k0i < k_hi && (k0i >= k_begin || k0i < kept)) ? sa[r] * scale_log2 : -INFINITY;
-        sc[4 + r] = (k1i <= qpos[qb] && k1i < k_hi && (k1i >= k_begin || k1i < kept)) ? sb[r] * scale_log2 : -INFINITY;
+        sc[r] = (k0i <= qpos[qb] && k0i < k_hi && (k0i >= k_begin || k0i < kept)) ? sa[r] * mul : -INFINITY;
+        sc[4 + r] = (k1i <= qpos[qb] && k1i < k_hi && (k1i >= k_begin || k1i < kept)) ? sb[r] * mul : -INFINITY;
         mx = fmaxf(mx, fmaxf(sc[r], sc[4 + r]));
       }
       mx = rows_max(mx);
@@ -291,17 +334,18 @@ __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
 // tile's loads in flight under the current tile's products): 64 queries per byte of K / V instead of 16.  K fragments are
 // 16-byte LDS reads, V^T fragments transposing LDS reads.  A wave whose columns end before the tile (causality) or lie past
 // the run's end only helps to load.
-template <int DT, int NSM, int NTM>
+template <int DT, int NSM, int NTM, bool BIASED>
 __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ seq_start, const int32_t* __restrict__ seq_first_pos, const uint16_t* __restrict__ sink,
     float scale_log2, uint16_t* __restrict__ out, int heads, int kv_heads, int dk, int dv, int64_t k_stride, int64_t v_stride,
-    int window, int shared_kv, int keep_first, int64_t out_stride) {
+    int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape) {
   constexpr int KSTR = NSM * 32 + 8, VSTR = NTM * 16 + 8;
   constexpr int KPASS = (32 * NSM * 4 + 255) / 256, VPASS = (32 * NTM * 2 + 255) / 256;  // 16-byte pieces per thread
   __shared__ __attribute__((aligned(16))) uint16_t lds_k[32 * KSTR];
   __shared__ __attribute__((aligned(16))) uint16_t lds_v[32 * VSTR];
+  __shared__ float lds_b[BIASED ? 96 : 1];   // the tile's biases by distance: 64 queries against 32 keys meet 95 distances
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t = lane & 15, c = lane >> 4;
   const int b = blockIdx.z;
   const int start = seq_start[b], count = seq_start[b + 1] - start, first = seq_first_pos[b];
@@ -378,7 +422,19 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
                 ? *reinterpret_cast<const Q4*>(v_cache + (int64_t)rv[u] * v_stride + (int64_t)g * dv + 8 * piece)  \
                 : Q4{0, 0, 0, 0};                                                                                  \
   }
+  // entry i of a tile's bias row: distance (first query - first key) - 31 + i
+  const float* bias_row = BIASED && shape.dist_bias ? shape.dist_bias + (int64_t)head * shape.dist_n : nullptr;
+  float br = 0.f;
+  auto bias_fetch = [&](int p) {
+    if constexpr (BIASED) {
+      if (bias_row && tid < 96) {
+        const int d = first + q0 - p - 31 + tid;
+        br = bias_row[d < 0 ? 0 : d < shape.dist_n ? d : shape.dist_n - 1];
+      }
+    }
+  };
 #define LL_STAGE()                                                                           \
+  if (BIASED && tid < 96) lds_b[tid] = br;                                                   \
   _Pragma("unroll") for (int u = 0; u < KPASS; ++u) {                                        \
     const int i = tid + 256 * u, key = i / kcpr, piece = i - key * kcpr;                     \
     if (key < 32) *reinterpret_cast<Q4*>(&lds_k[key * KSTR + 8 * piece]) = kr[u];            \
@@ -389,6 +445,7 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
   }
   LL_ROWS(k_first_wg)
   LL_FETCH(k_first_wg)
+  bias_fetch(k_first_wg);
   LL_ROWS(next_tile(k_first_wg))   // (past the range: nothing is read)
   __syncthreads();   // the zero fill is complete
   LL_STAGE()
@@ -397,6 +454,7 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
     p1 = next_tile(p0);
     if (p1 < k_hi) {
       LL_FETCH(p1)
+      bias_fetch(p1);
       LL_ROWS(next_tile(p1))
     }
     if (wave_on && p0 < k_hi_w && (p0 + 32 > k_lo_w || p0 < keep_first)) {
@@ -410,13 +468,22 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
           sb = mfma16<DT>(kb, qf[s], sb);
         }
       }
+      if constexpr (BIASED) {
+        const int at = 31 + (qi - q0) - 4 * c;   // bias entry of key p0 + 4 c (in 19 .. 94; 16 lower for the second half)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          sa[r] = shaped_score(sa[r], shape, lds_b[at - r]);
+          sb[r] = shaped_score(sb[r], shape, lds_b[at - 16 - r]);
+        }
+      }
+      const float mul = BIASED ? 1.0f : scale_log2;
       float sc[8];
       float mx = -INFINITY;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int k0i = p0 + 4 * c + r, k1i = k0i + 16;
-        sc[r] = (k0i <= qpos && (k0i >= wlo || k0i < keep_first)) ? sa[r] * scale_log2 : -INFINITY;
-        sc[4 + r] = (k1i <= qpos && (k1i >= wlo || k1i < keep_first)) ? sb[r] * scale_log2 : -INFINITY;
+        sc[r] = (k0i <= qpos && (k0i >= wlo || k0i < keep_first)) ? sa[r] * mul : -INFINITY;
+        sc[4 + r] = (k1i <= qpos && (k1i >= wlo || k1i < keep_first)) ? sb[r] * mul : -INFINITY;
         mx = fmaxf(mx, fmaxf(sc[r], sc[4 + r]));
       }
       mx = rows_max(mx);
@@ -527,7 +594,8 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
                                         const int32_t* seq_first_pos, const void* sink, float scale, void* out, int64_t n,
                                         int64_t batch, int64_t longest_run, int64_t longest_context, int decode, float* partials,
                                         int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv, int64_t k_stride, int64_t v_stride,
-                                        int64_t window, int64_t keep_first, int64_t out_stride, int dtype, void* stream) {
+                                        int64_t window, int64_t keep_first, int64_t out_stride, float cap, const float* dist_bias,
+                                        int64_t dist_n, int dtype, void* stream) {
   if (!ll_ragged_attention_mfma_supported(dk, dv, dtype)) return dtype == LL_F32 ? LL_ERR_DTYPE : LL_ERR_SHAPE;
   if (k_stride < kv_heads * dk || v_stride < kv_heads * dv || k_stride % 8 || v_stride % 8 || window < 0 || window > 0x7fffffff ||
       keep_first < 0 || keep_first > 0x7fffffff || out_stride < heads * dv ||
@@ -545,22 +613,31 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
   const dim3 grid((unsigned)max_parts, (unsigned)(kv_heads * ((group + 15) / 16)), (unsigned)batch);
   hipStream_t st = (hipStream_t)stream;
   const float scale_log2 = scale * kLog2e;
-#define CALL_D(DT, NS, NT)                                                                                                   \
-  ragged_attention_mfma_decode_kernel<DT, NS, NT><<<grid, 64, 0, st>>>(                                                      \
+  if (!(cap >= 0.f) || (dist_bias && (dist_n < 1 || dist_n > 0x7fffffff))) return LL_ERR_SHAPE;
+  const bool biased = cap > 0.f || dist_bias;
+  const ScoreShape shape = {scale, cap, dist_bias, dist_bias ? (int)dist_n : 1};
+#define CALL_DB(DT, NS, NT, B)                                                                                                   \
+  ragged_attention_mfma_decode_kernel<DT, NS, NT, B><<<grid, 64, 0, st>>>(                                                      \
       (const uint16_t*)q, (const uint16_t*)k_cache, (const uint16_t*)v_cache, token_table, tt_stride, seq_req, seq_start,    \
       seq_first_pos, (const uint16_t*)sink, scale_log2, (uint16_t*)out, partials, max_parts, (int)heads, (int)kv_heads, (int)dk, \
-      (int)dv, k_stride, v_stride, (int)window, shared_kv, (int)keep_first, out_stride)
+      (int)dv, k_stride, v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape)
+#define CALL_D(DT, NS, NT)                         \
+  if (biased) { CALL_DB(DT, NS, NT, true); }       \
+  else { CALL_DB(DT, NS, NT, false); }
 #define CALL(DT)                                         \
   if (dk <= 64 && dv <= 64) { CALL_D(DT, 2, 4); }        \
   else if (dk <= 128 && dv <= 128) { CALL_D(DT, 4, 8); } \
   else { CALL_D(DT, 8, 16); }
   if (!decode) {
     const dim3 grid4((unsigned)((longest_run + 63) / 64), (unsigned)heads, (unsigned)batch);
-#define CALL_4(DT, NS, NT)                                                                                                  \
-  ragged_attention_mfma_prefill4_kernel<DT, NS, NT><<<grid4, 256, 0, st>>>(                                                 \
+#define CALL_4B(DT, NS, NT, B)                                                                                                \
+  ragged_attention_mfma_prefill4_kernel<DT, NS, NT, B><<<grid4, 256, 0, st>>>(                                                 \
       (const uint16_t*)q, (const uint16_t*)k_cache, (const uint16_t*)v_cache, token_table, tt_stride, seq_req, seq_start,   \
       seq_first_pos, (const uint16_t*)sink, scale_log2, (uint16_t*)out, (int)heads, (int)kv_heads, (int)dk, (int)dv, k_stride,   \
-      v_stride, (int)window, shared_kv, (int)keep_first, out_stride)
+      v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape)
+#define CALL_4(DT, NS, NT)                         \
+  if (biased) { CALL_4B(DT, NS, NT, true); }       \
+  else { CALL_4B(DT, NS, NT, false); }
 #define CALL_P(DT)                                       \
   if (dk <= 64 && dv <= 64) { CALL_4(DT, 2, 4); }        \
   else if (dk <= 128 && dv <= 128) { CALL_4(DT, 4, 8); } \
@@ -568,11 +645,13 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
     if (dtype == LL_F16) { CALL_P(LL_F16) } else { CALL_P(LL_BF16) }
 #undef CALL_P
 #undef CALL_4
+#undef CALL_4B
     return LL_LAUNCH_CHECK();
   }
   if (dtype == LL_F16) { CALL(LL_F16) } else { CALL(LL_BF16) }
 #undef CALL
 #undef CALL_D
+#undef CALL_DB
   if (decode && max_parts > 1) {
     const int64_t waves = n * heads;
     if (dtype == LL_F16)

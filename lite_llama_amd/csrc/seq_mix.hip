@@ -12,6 +12,8 @@
 //                          lower-bounded forget gate and a per-head RMS norm of o (HGRN2), state in fp32 slots
 //   ll_mingru_scan         per-channel gated recurrence S_t = (1 - z_t) S_(t-1) + z_t c_t whose gates read the current token
 //                          only (minGRU), silu-gated read-out, state in fp32 slots
+//   ll_rglru_scan          per-channel real-gated recurrence S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t (RG-LRU), read-out times
+//                          the tanh form of gelu of a gate row, state in fp32 slots
 //
 // Storage dtype DT = LL_F16 / LL_BF16 / LL_F32 for activations and weights; everything that the recurrence, the norms and
 // the residual touch is fp32.  A step is described by   seq_start[b + 1] (first flat token of each sequence's run),
@@ -686,6 +688,133 @@ __global__ __launch_bounds__(256) void mingru_carry_kernel(int width, const int3
   if (count > 0) *slot = S;
 }
 
+// RG-LRU: per channel  r = sigmoid(r_raw + r_bias), i = sigmoid(i_raw + i_bias), log a = -8 r softplus(lam),
+// S_t = a S_(t-1) + sqrt(1 - a^2) i u_t, out = S_t * gelu(y_t).  r_raw and i_raw are the rows of a block-diagonal product: block p
+// of bs channels holds [r (bs) | i (bs)] at columns 2 p bs ..  1 - a^2 is taken as -expm1(2 log a): exact where a is close to 1.
+struct RglruArgs {
+  const void* u;        // [n][u_ld]
+  int64_t u_ld;
+  const void* gates;    // [n][g_ld]
+  int64_t g_ld;
+  const void* r_bias;   // [width]
+  const void* i_bias;
+  const void* lam;
+  const void* y;        // [n][y_ld]
+  int64_t y_ld;
+  void* out;            // [n][width]
+  int width, bs;
+  const int32_t* seq_start;
+  const int32_t* seq_first_pos;
+  const int32_t* seq_slot;
+  float* state;         // [slots][width]
+  int max_chunks;
+  float* scratch;       // chunk maps [batch * max_chunks][width][2]
+  float2* ab;           // (a, b) of every token and channel [n][width]
+};
+
+template <int DT>
+__device__ __forceinline__ float gelu_tanh_f32(float v) {
+  const float inner = 0.7978845608028654f * (v + 0.044715f * v * v * v);
+  float th;
+  if constexpr (DT == LL_F32) th = tanhf(inner);
+  else th = 2.0f * ll_sigmoidf(2.0f * inner) - 1.0f;
+  return 0.5f * v * (1.0f + th);
+}
+
+// what a channel's parameters contribute, once per thread
+struct RglruChannel {
+  float rb, ib, rate;   // rate = 8 softplus(lam)
+  int64_t r_at, i_at;   // columns of the two gates
+};
+template <int DT>
+__device__ __forceinline__ RglruChannel rglru_channel(const RglruArgs& a, int c) {
+  RglruChannel ch;
+  ch.rb = ldv<DT>(a.r_bias, c);
+  ch.ib = ldv<DT>(a.i_bias, c);
+  ch.rate = 8.0f * softplus_f32(ldv<DT>(a.lam, c));
+  const int p = c / a.bs;
+  ch.r_at = (int64_t)p * a.bs + c;
+  ch.i_at = ch.r_at + a.bs;
+  return ch;
+}
+template <int DT>
+__device__ __forceinline__ float2 rglru_step(const RglruChannel& ch, float rr, float ir, float u) {
+  const float r = 1.0f / (1.0f + expf(-(rr + ch.rb)));
+  const float i = 1.0f / (1.0f + expf(-(ir + ch.ib)));
+  const float la = -r * ch.rate;
+  return make_float2(expf(la), sqrtf(-expm1f(2.0f * la)) * (i * u));
+}
+
+// One thread per (sequence, channel) walks the run's tokens in order.
+template <int DT>
+__global__ __launch_bounds__(256) void rglru_scan_kernel(const RglruArgs a) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= a.width) return;
+  const int b = blockIdx.y;
+  const int start = a.seq_start[b], stop = a.seq_start[b + 1];
+  if (start >= stop) return;
+  float* slot = a.state + (int64_t)a.seq_slot[b] * a.width + c;
+  float S = a.seq_first_pos[b] > 0 ? *slot : 0.f;
+  const RglruChannel ch = rglru_channel<DT>(a, c);
+  auto update = [&](float rr, float ir, float uv, float yv, int64_t t) {
+    const float2 ab = rglru_step<DT>(ch, rr, ir, uv);
+    S = ab.x * S + ab.y;
+    stv<DT>(a.out, t * a.width + c, S * gelu_tanh_f32<DT>(yv));
+  };
+  int64_t t = start;
+  for (; t + 4 <= stop; t += 4) {   // the loads of four tokens are issued before the four dependent updates
+    float rr[4], ir[4], uv[4], yv[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      rr[k] = ldv<DT>(a.gates, (t + k) * a.g_ld + ch.r_at);
+      ir[k] = ldv<DT>(a.gates, (t + k) * a.g_ld + ch.i_at);
+      uv[k] = ldv<DT>(a.u, (t + k) * a.u_ld + c);
+      yv[k] = ldv<DT>(a.y, (t + k) * a.y_ld + c);
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) update(rr[k], ir[k], uv[k], yv[k], t + k);
+  }
+  for (; t < stop; ++t)
+    update(ldv<DT>(a.gates, t * a.g_ld + ch.r_at), ldv<DT>(a.gates, t * a.g_ld + ch.i_at), ldv<DT>(a.u, t * a.u_ld + c),
+           ldv<DT>(a.y, t * a.y_ld + c), t);
+  *slot = S;
+}
+
+// Long runs: chunks of kGruChunk tokens side by side as for the minGRU above (pass 1, mingru_carry_kernel, pass 3); pass 1 leaves
+// every token's (a, b) so that pass 3 evaluates no gate again.
+template <int DT, int PASS>
+__global__ __launch_bounds__(256) void rglru_chunk_kernel(const RglruArgs a) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= a.width) return;
+  const int b = blockIdx.y / a.max_chunks, k = blockIdx.y - b * a.max_chunks;
+  const int start = a.seq_start[b] + k * kGruChunk, stop_run = a.seq_start[b + 1];
+  if (start >= stop_run) return;
+  const int stop = start + kGruChunk < stop_run ? start + kGruChunk : stop_run;
+  float* rec = a.scratch + ((int64_t)blockIdx.y * a.width + c) * 2;
+  if (PASS == 1) {
+    const RglruChannel ch = rglru_channel<DT>(a, c);
+    float A = 1.0f, B = 0.f;
+#pragma unroll 4
+    for (int64_t t = start; t < stop; ++t) {
+      const float2 ab = rglru_step<DT>(ch, ldv<DT>(a.gates, t * a.g_ld + ch.r_at), ldv<DT>(a.gates, t * a.g_ld + ch.i_at),
+                                       ldv<DT>(a.u, t * a.u_ld + c));
+      a.ab[t * a.width + c] = ab;
+      A = ab.x * A;
+      B = ab.x * B + ab.y;
+    }
+    rec[0] = A;
+    rec[1] = B;
+  } else {
+    float S = rec[0];   // (the carry pass left the entering state here)
+#pragma unroll 4
+    for (int64_t t = start; t < stop; ++t) {
+      const float2 ab = a.ab[t * a.width + c];
+      S = ab.x * S + ab.y;
+      stv<DT>(a.out, t * a.width + c, S * gelu_tanh_f32<DT>(ldv<DT>(a.y, t * a.y_ld + c)));
+    }
+  }
+}
+
 }  // namespace
 
 #define LL_BY_DTYPE(dtype, CALL)             \
@@ -872,6 +1001,50 @@ extern "C" int ll_mingru_scan(const void* z, const void* x, const void* g, int64
   const dim3 grid((unsigned)((width + 255) / 256), (unsigned)batch);
 #define CALL(DT) \
   mingru_scan_kernel<DT><<<grid, 256, 0, st>>>(z, x, g, ld, z_bias, x_bias, out, (int)width, seq_start, seq_first_pos, seq_slot, state)
+  LL_BY_DTYPE(dtype, CALL);
+#undef CALL
+  return LL_LAUNCH_CHECK();
+}
+
+// floats of the scratch for long runs (0: the plain walk): chunk maps, then (a, b) per token and channel
+extern "C" int64_t ll_rglru_scan_scratch_floats(int64_t n, int64_t batch, int64_t width, int64_t longest_run) {
+  const int64_t maps = ll_mingru_scan_scratch_floats(batch, width, longest_run);
+  return maps ? maps + 2 * n * width : 0;
+}
+
+extern "C" int ll_rglru_scan(const void* u, int64_t u_ld, const void* gates, int64_t g_ld, const void* r_bias, const void* i_bias,
+                             const void* lam, const void* y, int64_t y_ld, void* out, int64_t n, int64_t batch, int64_t width,
+                             int64_t blocks, const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot,
+                             float* state, int64_t longest_run, float* scratch, int dtype, void* stream) {
+  if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
+  if (n < 0 || batch < 0 || batch > 65535 || width < 1 || width > (1 << 24) || blocks < 1 || width % blocks || u_ld < width ||
+      g_ld < 2 * width || y_ld < width || longest_run < 0)
+    return LL_ERR_SHAPE;
+  if (n == 0 || batch == 0) return LL_OK;
+  if (!u || !gates || !r_bias || !i_bias || !lam || !y || !out || !seq_start || !seq_first_pos || !seq_slot || !state) return LL_ERR_ARG;
+  hipStream_t st = (hipStream_t)stream;
+  RglruArgs a;
+  a.u = u; a.u_ld = u_ld; a.gates = gates; a.g_ld = g_ld; a.r_bias = r_bias; a.i_bias = i_bias; a.lam = lam; a.y = y; a.y_ld = y_ld;
+  a.out = out; a.width = (int)width; a.bs = (int)(width / blocks); a.seq_start = seq_start; a.seq_first_pos = seq_first_pos;
+  a.seq_slot = seq_slot; a.state = state; a.max_chunks = 0; a.scratch = nullptr; a.ab = nullptr;
+  const int64_t max_chunks = (longest_run + kGruChunk - 1) / kGruChunk;
+  const int64_t maps = scratch ? ll_mingru_scan_scratch_floats(batch, width, longest_run) : 0;
+  const unsigned cols = (unsigned)((width + 255) / 256);
+  if (maps > 0 && batch * max_chunks <= 65535) {
+    a.max_chunks = (int)max_chunks;
+    a.scratch = scratch;
+    a.ab = reinterpret_cast<float2*>(scratch + maps);
+    const dim3 grid_c(cols, (unsigned)(batch * max_chunks)), grid_b(cols, (unsigned)batch);
+#define CALL(DT)                                                                                                                 \
+  rglru_chunk_kernel<DT, 1><<<grid_c, 256, 0, st>>>(a);                                                                          \
+  mingru_carry_kernel<<<grid_b, 256, 0, st>>>((int)width, seq_start, seq_first_pos, seq_slot, state, (int)max_chunks, scratch);  \
+  rglru_chunk_kernel<DT, 2><<<grid_c, 256, 0, st>>>(a)
+    LL_BY_DTYPE(dtype, CALL);
+#undef CALL
+    return LL_LAUNCH_CHECK();
+  }
+  const dim3 grid(cols, (unsigned)batch);
+#define CALL(DT) rglru_scan_kernel<DT><<<grid, 256, 0, st>>>(a)
   LL_BY_DTYPE(dtype, CALL);
 #undef CALL
   return LL_LAUNCH_CHECK();

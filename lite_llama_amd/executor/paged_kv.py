@@ -97,8 +97,8 @@ class PagedStateCache(PagedKVPool):
     """Cache of a model whose layer RUNS differ in what they keep per sequence (a layer that runs several times in a forward
     pass keeps one set per run): attention runs own ``(K [rows, kv_heads, dk], V [rows, kv_heads, dv])`` in the block pool --
     key and value widths may differ --, latent-attention runs one row ``[latent | rotated key part]`` per token, recurrent runs own a fixed-size fp32 state ``[slots, heads, dk, dv]``, and any run may
-    own a token-shift row pair ``[2, slots, width]`` (double-buffered by the sequence's parity).  An attention run with a short
-    convolution in front of it carries the projected rows of a sequence's last positions, ``[2, slots, taps - 1, channels]``,
+    own a token-shift row pair ``[2, slots, width]`` (double-buffered by the sequence's parity).  A run with a short
+    convolution in front of it (attention or recurrence) carries the projected rows of a sequence's last positions, ``[2, slots, taps - 1, channels]``,
     double-buffered the same way; a run whose values are blended with those of an earlier run names that run in
     ``value_source``; a model whose input depends on the previous token keeps it per sequence in ``prev_token [2, slots]``.  One block allocator, one
     block table and one per-token row table serve all attention runs; a sequence's slot is its row of those tables, so blocks
@@ -108,8 +108,8 @@ class PagedStateCache(PagedKVPool):
     def __init__(self, runs, num_blocks: int, block_size: int, device, max_requests: int, max_seq_len: int, dtype,
                  previous_token: bool = False):
         """``runs``: one mapping per layer run: ``{"kind": "attention", "kv_heads", "dk", "dv"}``, ``{"kind": "latent", "rank",
-        "rot"}`` or ``{"kind": "recurrent", "heads", "dk", "dv"}``, each with an optional ``"shift_width"``; attention runs may
-        add ``"conv_taps"`` / ``"conv_channels"`` (rows carried for a convolution of that many taps), ``"value_mix": True``
+        "rot"}`` or ``{"kind": "recurrent", "heads", "dk", "dv"}``, each with an optional ``"shift_width"``; attention and recurrent runs
+        may add ``"conv_taps"`` / ``"conv_channels"`` (rows carried for a convolution of that many taps), attention runs ``"value_mix": True``
         (the first such run is the value source of the later ones) and ``"state": (heads, dk, dv)`` (a recurrence that runs
         beside the attention keeps its fp32 state in the same run).  ``previous_token``: keep each sequence's last token."""
         self.runs = [dict(r) for r in runs]
@@ -123,7 +123,7 @@ class PagedStateCache(PagedKVPool):
         buffers = []
         first_mix = None
         for index, r in enumerate(self.runs):
-            taps = int(r.get("conv_taps", 0)) if r["kind"] == "attention" else 0
+            taps = int(r.get("conv_taps", 0))
             self.conv.append(torch.zeros(2, slots, taps - 1, int(r["conv_channels"]), dtype=dtype, device=dev) if taps > 1 else None)
             mixes = r["kind"] == "attention" and bool(r.get("value_mix"))
             self.value_source.append(first_mix if mixes else None)

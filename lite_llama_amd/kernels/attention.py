@@ -409,13 +409,15 @@ def rownorm_rope_cache(qkv, heads: int, kv_heads: int, dk: int, dv: int, step, k
 
 @torch.no_grad()
 def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=None, window: int = 0, keep_first: int = 0,
-                     out=None):
+                     out=None, cap: float = 0.0, dist_bias=None):
     """Causal softmax attention of every token of a ragged step against positions ``0 .. its own`` of its sequence, keys and
     values read through ``token_table[request][position]``; ``sink [heads]`` adds ``exp(sink_h)`` to each head's denominator;
     ``window > 0`` keeps the last ``window`` positions (the token's own included) and, besides them, the sequence's first
     ``keep_first`` positions.  ``k_cache [rows, kv_heads, dk]`` /
     ``v_cache [rows, kv_heads, dv]`` may be row-strided views (the values of a latent cache are a column range of its key
-    rows).  Scores, weights and the output sum are fp32.  Returns ``[n, heads * dv]`` (``out``: a view of that shape with a
+    rows).  ``cap > 0``: scaled scores become ``cap tanh(score / cap)``; ``dist_bias`` (fp32 ``[heads, m]``): then the entry of the
+    distance between token and key is added per head (distances from ``m - 1`` on read the last entry).  Scores, weights and the
+    output sum are fp32.  Returns ``[n, heads * dv]`` (``out``: a view of that shape with a
     unit inner stride, e.g. a column range of the next projection's input)."""
     L.require_cuda(q, k_cache, v_cache, token_table)
     n, heads, dk = q.shape
@@ -430,6 +432,10 @@ def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=
         raise ValueError("ragged_attention: the token table is row-major int32")
     if sink is not None and (sink.dtype != dt or sink.numel() != heads or not sink.is_contiguous()):
         raise ValueError("ragged_attention: sink is [heads] in the queries' dtype")
+    if dist_bias is not None and (dist_bias.dtype != torch.float32 or dist_bias.dim() != 2 or dist_bias.shape[0] != heads
+                                  or dist_bias.shape[1] < 1 or not dist_bias.is_contiguous() or not dist_bias.is_cuda):
+        raise ValueError("ragged_attention: the distance bias is fp32 [heads, distances]")
+    bias_n = dist_bias.shape[1] if dist_bias is not None else 0
     if step.num_tokens != n:
         raise ValueError("ragged_attention: the step describes another number of tokens")
     ks, vs = k_cache.stride(0), v_cache.stride(0)
@@ -452,12 +458,14 @@ def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=
             q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), token_table.data_ptr(), token_table.stride(0),
             step.seq_req.data_ptr(), step.seq_start.data_ptr(), step.seq_first_pos.data_ptr(), L.ptr(sink), float(scale),
             out.data_ptr(), n, step.num_seqs, step.longest_run, step.longest_context, 1 if decode else 0, L.ptr(scratch), heads,
-            kv_heads, dk, dv, ks, vs, int(window), int(keep_first), os_, L.dtype_code(dt), L.stream_ptr()), "ragged_attention_mfma")
+            kv_heads, dk, dv, ks, vs, int(window), int(keep_first), os_, float(cap), L.ptr(dist_bias), bias_n, L.dtype_code(dt),
+            L.stream_ptr()), "ragged_attention_mfma")
         return out
     L.check(L.lib().ll_ragged_attention(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), token_table.data_ptr(),
                                         token_table.stride(0), step.seq_req.data_ptr(), step.tok_seq.data_ptr(),
                                         step.tok_pos.data_ptr(), L.ptr(sink), float(scale), out.data_ptr(), n, heads, kv_heads, dk,
-                                        dv, ks, vs, int(window), int(keep_first), os_, L.dtype_code(dt), L.stream_ptr()),
+                                        dv, ks, vs, int(window), int(keep_first), os_, float(cap), L.ptr(dist_bias), bias_n,
+                                        L.dtype_code(dt), L.stream_ptr()),
             "ragged_attention")
     return out
 

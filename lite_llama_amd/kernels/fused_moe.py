@@ -263,7 +263,8 @@ def group_router(h: torch.Tensor, router_weight: torch.Tensor, top: int, group_c
     correction[e]`` (``correction [experts]`` in the storage dtype, or ``None``) and weighted by their scores alone, not
     renormalised.  The last ``identity`` router outputs stand for experts that return the token's own row: their slots keep
     ids ``>= experts - identity`` (which :func:`sparse_glu_experts` leaves as zero rows) and ``extra`` is the sum of their
-    scores per token -- the factor of ``h`` itself in the sublayer's result."""
+    scores per token -- the factor of ``h`` itself in the sublayer's result.  ``scoring="sigmoid_plain"``: as ``"sigmoid"``, but the
+    weights are the chosen scores themselves (times ``route_scale``), not divided by their sum."""
     L.require_cuda(h, router_weight, extra_weight, correction)
     n, width = h.shape
     experts = router_weight.shape[0]
@@ -281,11 +282,24 @@ def group_router(h: torch.Tensor, router_weight: torch.Tensor, top: int, group_c
     logits = torch.empty(n, experts + (1 if extra_weight is not None else 0), dtype=torch.float32, device=h.device)
     L.check(L.lib().ll_group_router(h.data_ptr(), h.stride(0), router_weight.data_ptr(), L.ptr(extra_weight), n, width, experts,
                                     int(top), int(group_count), int(group_keep), float(route_scale),
-                                    {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2}[scoring], ids.data_ptr(),
+                                    {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2, "sigmoid_plain": 3}[scoring], ids.data_ptr(),
                                     weights.data_ptr(), L.ptr(extra), logits.data_ptr(), L.ptr(correction), int(identity),
                                     L.dtype_code(h.dtype), L.stream_ptr()),
             "group_router")
     return ids, weights, extra
+
+
+def _sort_slots(ids: torch.Tensor, slots: int, experts: int, width: int, ff: int, dt):
+    """Slots sorted by expert in row blocks: ``(rows per block, sorted slots, expert of every block, [padded count])``."""
+    lib = L.lib()
+    block = int(lib.ll_moe_rows_block(slots, experts, width, ff, L.dtype_code(dt)))
+    padded = slots + experts * (block - 1)
+    meta = torch.empty(experts + padded + -(-padded // block) + 1, dtype=torch.int32, device=ids.device)
+    counts, sorted_ids = meta[:experts], meta[experts:experts + padded]
+    block_expert, num_post = meta[experts + padded:-1], meta[-1:]
+    L.check(lib.ll_moe_sort(ids.data_ptr(), slots, experts, block, counts.data_ptr(), sorted_ids.data_ptr(), block_expert.data_ptr(),
+                            num_post.data_ptr(), L.stream_ptr()), "moe_sort")
+    return block, sorted_ids, block_expert, num_post
 
 
 @torch.no_grad()
@@ -311,13 +325,7 @@ def sparse_glu_experts(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.T
         raise ValueError("sparse_glu_experts: int32 ids and fp32 weights [n, top]")
     lib = L.lib()
     slots = n * top
-    block = int(lib.ll_moe_rows_block(slots, experts, width, ff, L.dtype_code(dt)))
-    padded = slots + experts * (block - 1)
-    meta = torch.empty(experts + padded + -(-padded // block) + 1, dtype=torch.int32, device=h.device)
-    counts, sorted_ids = meta[:experts], meta[experts:experts + padded]
-    block_expert, num_post = meta[experts + padded:-1], meta[-1:]
-    L.check(lib.ll_moe_sort(ids.data_ptr(), slots, experts, block, counts.data_ptr(), sorted_ids.data_ptr(), block_expert.data_ptr(),
-                            num_post.data_ptr(), L.stream_ptr()), "moe_sort")
+    block, sorted_ids, block_expert, num_post = _sort_slots(ids, slots, experts, width, ff, dt)
     act = torch.empty(slots, ff, dtype=dt, device=h.device)
     out = (torch.zeros if skipped_ids else torch.empty)(n, top, width, dtype=dt, device=h.device)
     code, st = L.dtype_code(dt), L.stream_ptr()
@@ -328,4 +336,36 @@ def sparse_glu_experts(h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.T
     L.check(lib.ll_moe_rows_gemm(act.data_ptr(), ff, 1, w_down.data_ptr(), w_down.stride(0), ff, width, 0, weights.data_ptr(),
                                  out.data_ptr(), width, sorted_ids.data_ptr(), block_expert.data_ptr(), num_post.data_ptr(), slots,
                                  experts, block, 0.0, code, st), "moe_rows_gemm (down)")
+    return out
+
+
+@torch.no_grad()
+def sparse_square_experts(h: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor,
+                          weights: torch.Tensor) -> torch.Tensor:
+    """Per slot (token, k): ``down_e(relu(up_e (weights * h))^2)`` with ``e = ids[token, k]`` -- experts without a gate, whose weight
+    multiplies their INPUT (it is applied to the fp32 sums of the first product, which are linear in the input).  ``w_up
+    [experts, ff, width]``, ``w_down [experts, width, ff]``.  Returns the slots' rows ``[n, top, width]`` in the storage dtype (their
+    sum over k is the caller's).  Slots are sorted by expert on the device; every product accumulates in fp32."""
+    L.require_cuda(h, w_up, w_down, ids, weights)
+    n, width = h.shape
+    experts, ff, _ = w_up.shape
+    top, dt = ids.shape[1], h.dtype
+    if (not h.is_contiguous() or w_up.dtype != dt or w_down.dtype != dt or not w_up.is_contiguous() or not w_down.is_contiguous()
+            or w_up.shape[2] != width or tuple(w_down.shape) != (experts, width, ff)):
+        raise ValueError("sparse_square_experts: h [n, width], up [E, ff, width], down [E, width, ff] of one dtype")
+    if ids.dtype != torch.int32 or weights.dtype != torch.float32 or not ids.is_contiguous() or not weights.is_contiguous() \
+            or weights.shape != ids.shape:
+        raise ValueError("sparse_square_experts: int32 ids and fp32 weights [n, top]")
+    lib = L.lib()
+    slots = n * top
+    block, sorted_ids, block_expert, num_post = _sort_slots(ids, slots, experts, width, ff, dt)
+    act = torch.empty(slots, ff, dtype=dt, device=h.device)
+    out = torch.empty(n, top, width, dtype=dt, device=h.device)
+    code, st = L.dtype_code(dt), L.stream_ptr()
+    L.check(lib.ll_moe_rows_gemm(h.data_ptr(), h.stride(0), top, w_up.data_ptr(), w_up.stride(0), width, ff, 3, weights.data_ptr(),
+                                 act.data_ptr(), ff, sorted_ids.data_ptr(), block_expert.data_ptr(), num_post.data_ptr(), slots,
+                                 experts, block, 0.0, code, st), "moe_rows_gemm (up)")
+    L.check(lib.ll_moe_rows_gemm(act.data_ptr(), ff, 1, w_down.data_ptr(), w_down.stride(0), ff, width, 0, 0, out.data_ptr(), width,
+                                 sorted_ids.data_ptr(), block_expert.data_ptr(), num_post.data_ptr(), slots, experts, block, 0.0, code,
+                                 st), "moe_rows_gemm (down)")
     return out

@@ -573,6 +573,18 @@ def glu_act(gate: torch.Tensor, ff: int, kind: str, up: torch.Tensor | None = No
 
 
 @torch.no_grad()
+def relu_square(x: torch.Tensor, ff: int) -> torch.Tensor:
+    """``relu(x[:, :ff])^2`` of row-strided rows (fp32 arithmetic, one rounding to the storage dtype)."""
+    L.require_cuda(x)
+    if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] < ff:
+        raise ValueError("relu_square: rows are [n, >= ff] with a unit inner stride")
+    out = torch.empty(x.shape[0], ff, dtype=x.dtype, device=x.device)
+    L.check(L.lib().ll_glu_act(out.data_ptr(), ff, x.data_ptr(), max(x.stride(0), ff), 0, 0, x.shape[0], int(ff), 4, 0.0, 0.0,
+                               L.dtype_code(x.dtype), L.stream_ptr()), "relu_square")
+    return out
+
+
+@torch.no_grad()
 def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
     """``x <- cap * tanh(x / cap)`` in place (fp32 arithmetic)."""
     L.require_cuda(x)
@@ -580,3 +592,61 @@ def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
         raise ValueError("softcap_: a contiguous tensor")
     L.check(L.lib().ll_softcap(x.data_ptr(), x.numel(), float(cap), L.dtype_code(x.dtype), L.stream_ptr()), "softcap")
     return x
+
+
+# ------------------------------------------------------------------------------------- #
+# several mixed residual streams (csrc/stream_norm.hip)
+# ------------------------------------------------------------------------------------- #
+class StreamUpdate:
+    """A sublayer's result that has not entered the residual streams yet: ``y [n, parts, width]`` (the parts are summed), optionally
+    ``+ shared_scale[t] * shared[t]``, times ``scale [width]``, to be added to stream ``t`` times ``out[t]`` while the streams are mixed
+    by ``mix [from, to]``."""
+
+    __slots__ = ("y", "scale", "mix", "out", "shared", "shared_scale")
+
+    def __init__(self, y, scale, mix, out, shared=None, shared_scale=None):
+        self.y = y if y.dim() == 3 else y.unsqueeze(1)
+        self.scale, self.mix, self.out, self.shared, self.shared_scale = scale, mix, out, shared, shared_scale
+
+    def rows(self, index: torch.Tensor) -> "StreamUpdate":
+        """The update of the listed tokens only."""
+        pick = lambda t: None if t is None else t[index].contiguous()  # noqa: E731
+        return StreamUpdate(pick(self.y), self.scale, self.mix, self.out, pick(self.shared), pick(self.shared_scale))
+
+
+@torch.no_grad()
+def stream_norm(x: torch.Tensor, update: "StreamUpdate | None", streams: int, gather, weight, eps: float, weight_base: float = 0.0):
+    """``x``: the fp32 residual streams ``[n, streams, width]``, or one row per token ``[n, width]`` that every stream starts from.  The
+    pending ``update`` (or ``None``) enters and mixes the streams; then ``h = rmsnorm(sum_s gather[s] x_s) * (weight_base + weight)`` in
+    the storage dtype (``gather=None``: the plain sum; ``weight=None``: no ``h``).  One launch; everything fp32 until ``h``'s one
+    rounding.  Returns ``(h, x)``: ``x`` updated in place where it holds the streams, a new tensor where it was one row per token."""
+    L.require_cuda(x, gather, weight)
+    n, width = x.shape[0], x.shape[-1]
+    one = x.dim() == 2
+    if x.dtype != torch.float32 or not x.is_contiguous() or not (one or (x.dim() == 3 and x.shape[1] == streams)):
+        raise ValueError("stream_norm: the streams are contiguous fp32 [n, streams, width] (or [n, width] at the start)")
+    u = update
+    if u is None and weight is None:
+        return None, x
+    dt = weight.dtype if weight is not None else u.y.dtype
+    if weight is not None and (weight.numel() != width or not weight.is_contiguous()):
+        raise ValueError("stream_norm: the norm weight has one entry per channel")
+    if gather is not None and (gather.dtype != dt or gather.numel() != streams or not gather.is_contiguous()):
+        raise ValueError("stream_norm: one gather weight per stream, in the storage dtype")
+    args, out = (0, 0, 0, 0, 0, 0, 0), None
+    if u is not None:
+        if u.y.dtype != dt or u.y.shape[0] != n or u.y.shape[2] != width or not u.y.is_contiguous():
+            raise ValueError("stream_norm: the update is [n, parts, width] in the storage dtype")
+        if u.shared is not None and (u.shared.dtype != dt or u.shared.shape != (n, width) or not u.shared.is_contiguous()
+                                     or u.shared_scale.dtype != torch.float32 or u.shared_scale.numel() != n):
+            raise ValueError("stream_norm: the shared row is [n, width], its scale fp32 [n]")
+        for t, size in ((u.scale, width), (u.mix, streams * streams), (u.out, streams)):
+            if t is not None and (t.dtype != dt or t.numel() != size or not t.is_contiguous()):
+                raise ValueError("stream_norm: scale [width], mix [streams, streams] and out [streams] in the storage dtype")
+        out = torch.empty(n, streams, width, dtype=torch.float32, device=x.device) if one else x
+        args = (u.y.data_ptr(), u.y.shape[1], L.ptr(u.shared), L.ptr(u.shared_scale), L.ptr(u.scale), u.mix.data_ptr(), u.out.data_ptr())
+    h = torch.empty(n, width, dtype=dt, device=x.device) if weight is not None else None
+    L.check(L.lib().ll_stream_norm(x.data_ptr(), width if one else streams * width, 0 if one else width, L.ptr(out), *args, L.ptr(gather),
+                                   L.ptr(weight), float(weight_base), float(eps), L.ptr(h), n, width, int(streams), L.dtype_code(dt),
+                                   L.stream_ptr()), "stream_norm")
+    return h, (out if out is not None else x)

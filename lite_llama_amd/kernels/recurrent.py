@@ -78,6 +78,85 @@ def mingru_scan(zxg: torch.Tensor, width: int, z_bias, x_bias, step, state: torc
     return out
 
 
+@torch.no_grad()
+def rglru_scan(u: torch.Tensor, gates: torch.Tensor, r_bias, i_bias, lam, y: torch.Tensor, step, state: torch.Tensor) -> torch.Tensor:
+    """RG-LRU over a ragged step: per channel ``r = sigmoid(r_raw + r_bias)``, ``i = sigmoid(i_raw + i_bias)``,
+    ``log a = -8 r softplus(lam)``, ``S <- a S + sqrt(1 - a^2) i u``; returns ``S * gelu(y)`` (tanh form) ``[n, width]`` in the
+    storage dtype.  ``u [n, width]``, ``y [n, >= width]`` (row-strided views); ``gates [n, parts, 2, width / parts]``: the raw gates of
+    a block-diagonal product, ``r`` and ``i`` of a part side by side.  ``state [slots, width]`` fp32: a sequence whose run starts at
+    position 0 starts from zeros, every run leaves its final state.  Gates, decays and the state are fp32."""
+    L.require_cuda(u, gates, r_bias, i_bias, lam, y, state)
+    (n, width), dt = u.shape, u.dtype
+    if u.stride(1) != 1 or y.dim() != 2 or y.stride(1) != 1 or y.shape[0] != n or y.shape[1] < width or y.dtype != dt:
+        raise ValueError("rglru_scan: u [n, width] and y [n, >= width] of one dtype with unit inner strides")
+    if gates.dtype != dt or gates.dim() != 4 or gates.shape[0] != n or gates.shape[2] != 2 or gates.shape[1] * gates.shape[3] != width \
+            or not gates.is_contiguous():
+        raise ValueError("rglru_scan: contiguous gates [n, parts, 2, width / parts] in the rows' dtype")
+    for b in (r_bias, i_bias, lam):
+        if b.dtype != dt or b.numel() != width or not b.is_contiguous():
+            raise ValueError("rglru_scan: gate biases and lam have one entry per channel, in the rows' dtype")
+    if state.dtype != torch.float32 or not state.is_contiguous() or state.dim() != 2 or state.shape[1] != width:
+        raise ValueError("rglru_scan: state is contiguous fp32 [slots, width]")
+    if step.num_tokens != n:
+        raise ValueError("rglru_scan: the step describes another number of tokens")
+    out = torch.empty(n, width, dtype=dt, device=u.device)
+    floats = int(L.lib().ll_rglru_scan_scratch_floats(n, step.num_seqs, width, step.longest_run))
+    scratch = torch.empty(floats, dtype=torch.float32, device=u.device) if floats else None
+    L.check(L.lib().ll_rglru_scan(u.data_ptr(), max(u.stride(0), width), gates.data_ptr(), 2 * width, r_bias.data_ptr(), i_bias.data_ptr(),
+                                  lam.data_ptr(), y.data_ptr(), max(y.stride(0), width), out.data_ptr(), n, step.num_seqs, width,
+                                  gates.shape[1], step.seq_start.data_ptr(), step.seq_first_pos.data_ptr(), step.seq_slot.data_ptr(),
+                                  state.data_ptr(), step.longest_run, L.ptr(scratch), L.dtype_code(dt), L.stream_ptr()), "rglru_scan")
+    return out
+
+
+# ------------------------------------------------------------------------------------- #
+# gated delta rule (csrc/delta_scan.hip)
+# ------------------------------------------------------------------------------------- #
+def delta_scan_supported(dk: int, dv: int) -> bool:
+    return bool(L.lib().ll_delta_scan_supported(dk, dv))
+
+
+@torch.no_grad()
+def delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: int, dk: int, dv: int, step, state: torch.Tensor, *,
+               gate: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, beta: torch.Tensor, qk_heads: int | None = None,
+               q_scale: float = 1.0, unit_eps: float = 1e-6) -> torch.Tensor:
+    """Gated delta rule over a ragged step: per head ``S <- diag(g_t) S``, ``u = b_t (v_t - S^T k_t)``, ``S <- S + k_t u^T``,
+    ``o_t = S^T q_t``.  ``q`` / ``k`` (``qk_heads`` heads of ``dk`` shared by neighbouring value heads) and ``v`` (``heads`` of ``dv``) are
+    row-strided views; q and k heads are divided by ``sqrt(sum of squares + unit_eps)``, q also times ``q_scale``.  Per key entry
+    ``g = exp(-exp(a_log_h) softplus(gate + dt_bias))`` (``gate [n, heads dk]``), per head ``b = sigmoid(beta)`` (``beta [n, heads]``).
+    ``state [slots, heads, dk, dv]`` fp32: a sequence whose run starts at position 0 starts from zeros, every run leaves its final
+    state.  Unit norms, decays, step sizes, state and read-out are fp32.  Returns ``o`` fp32 ``[n, heads dv]``."""
+    L.require_cuda(q, k, v, state, gate, dt_bias, a_log, beta)
+    n, st = q.shape[0], q.dtype
+    qk_heads = heads if qk_heads is None else qk_heads
+    if qk_heads < 1 or heads % qk_heads:
+        raise ValueError(f"delta_scan: {heads} value heads do not divide over {qk_heads} query / key heads")
+    for t, cols, what in ((q, qk_heads * dk, "query"), (k, qk_heads * dk, "key"), (v, heads * dv, "value"), (gate, heads * dk, "decay logit"),
+                          (beta, heads, "step size")):
+        if t.dim() != 2 or t.stride(1) != 1 or t.shape[1] < cols or t.shape[0] != n or t.dtype != st:
+            raise ValueError(f"delta_scan: {what} rows are [n, >= {cols}] of the queries' dtype with a unit inner stride")
+    for t, size, what in ((dt_bias, heads * dk, "dt_bias"), (a_log, heads, "a_log")):
+        if t.dtype != st or t.numel() != size or not t.is_contiguous():
+            raise ValueError(f"delta_scan: {what} has {size} entries in the rows' dtype")
+    if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (heads, dk, dv):
+        raise ValueError("delta_scan: state is contiguous fp32 [slots, heads, dk, dv]")
+    if step.num_tokens != n:
+        raise ValueError("delta_scan: the step describes another number of tokens")
+    if not delta_scan_supported(dk, dv):
+        raise ValueError(f"delta_scan: head geometry {dk} x {dv} is not served (dk <= 256)")
+    o = torch.empty(n, heads * dv, dtype=torch.float32, device=q.device)
+    # runs of several tokens: decays and per-token scalars once, ahead of the walk; decode steps evaluate them in the walk
+    scratch = (torch.empty(int(L.lib().ll_delta_scan_scratch_floats(n, heads, dk)), dtype=torch.float32, device=q.device)
+               if step.longest_run != 1 else None)
+    ld = lambda t: max(t.stride(0), t.shape[1])  # noqa: E731  (one row: its stride means nothing)
+    L.check(L.lib().ll_delta_scan(q.data_ptr(), ld(q), k.data_ptr(), ld(k), v.data_ptr(), ld(v), heads, dk, dv, heads // qk_heads,
+                                  float(q_scale), float(unit_eps), gate.data_ptr(), ld(gate), dt_bias.data_ptr(), a_log.data_ptr(),
+                                  beta.data_ptr(), ld(beta), o.data_ptr(), step.num_seqs, step.seq_start.data_ptr(),
+                                  step.seq_first_pos.data_ptr(), step.seq_slot.data_ptr(), state.data_ptr(), L.ptr(scratch), n,
+                                  int(step.longest_run), L.dtype_code(st), L.stream_ptr()), "delta_scan")
+    return o
+
+
 # ------------------------------------------------------------------------------------- #
 # linear attention with a decay (csrc/linear_mix.hip)
 # ------------------------------------------------------------------------------------- #
@@ -194,8 +273,9 @@ def gated_out_norm(o: torch.Tensor, weight: torch.Tensor | None, eps: float, *, 
 
 
 @torch.no_grad()
-def conv_act(rows: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, step, state: torch.Tensor | None) -> torch.Tensor:
-    """``silu(bias + causal convolution)`` per channel over a ragged step: ``rows [n, channels]`` (a row-strided view),
+def conv_act(rows: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, step, state: torch.Tensor | None,
+             act: str | None = "silu") -> torch.Tensor:
+    """``act(bias + causal convolution)`` per channel (``act``: silu, or ``None``) over a ragged step: ``rows [n, channels]`` (a row-strided view),
     ``weight [channels, taps]`` (the last column is the current token's; zeros in front of position 0).  ``state
     [2, slots, taps - 1, channels]`` in the rows' dtype carries the raw rows of a sequence's last positions (the half named by
     the sequence's parity is read, the other written).  fp32 sums; returns ``[n, channels]`` in the rows' dtype."""
@@ -215,5 +295,5 @@ def conv_act(rows: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None
                                 channels, taps, L.ptr(state) if taps > 1 else 0, state[0].numel() if taps > 1 else 0,
                                 step.tok_seq.data_ptr(), step.tok_pos.data_ptr(), step.seq_start.data_ptr(),
                                 step.seq_first_pos.data_ptr(), step.seq_slot.data_ptr(), step.seq_parity.data_ptr(), n,
-                                L.dtype_code(dt), L.stream_ptr()), "conv_act")
+                                {None: 0, "silu": 1}[act], L.dtype_code(dt), L.stream_ptr()), "conv_act")
     return out

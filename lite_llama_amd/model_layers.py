@@ -29,6 +29,14 @@ description, out of mixers that take a ragged step (executor/ragged.py) and keep
   * :class:`BiasedGatedMLP`    ``down(silu(gate h + b) * (up h + b)) + b``
   * :class:`CorrectedSoftmaxMoE`  softmax scores over all router outputs, experts chosen by score + correction and weighted by
                                the score alone, clamped expert activations, router outputs that stand for "the input itself"
+  * :class:`BiasedDistanceAttention`  biased q / k / v, per-head q / k RMS norm, capped scores, a learned bias per head and distance
+                               bucket instead of a rotation (kernels/attention.py)
+  * :class:`ChannelDeltaMixer`  gated delta rule: q / k / v behind a short convolution, unit q / k heads, a decay per key entry from
+                               a low-rank projection, a state that is corrected towards the token's value (kernels/recurrent.py)
+  * :class:`RealGatedLRU`      a per-channel recurrence behind a convolution whose two gates are block-diagonal products, times a
+                               gelu branch (kernels/recurrent.py)
+  * :class:`SquareMoE`         sigmoid scores that multiply the experts' inputs (not renormalised), experts ``down(relu(up h)^2)``, a
+                               shared expert of the same form with a per-token scale
 
 The residual stream is fp32 throughout; every layer's residual add is fused into the norm that follows it
 (kernels/norm_act.py::add_rmsnorm_shift, which also applies the token shift in front of a mixer; or
@@ -36,8 +44,9 @@ kernels/norm_act.py::gated_group_norm for layers that wrap each sublayer in two 
 Projections run through the framework's linear layers (library GEMM for unquantised weights), with everything that reads one
 input fused into one launch at load time.  Families: Rakevik (``"architecture": "Rakevik"``: :class:`MixerLayer`),
 Rukedra (:class:`SandwichLayer`), Fekanex (:class:`ParallelLayer`: one norm per layer, mixer and feed-forward read its
-output side by side, and -- with a dense feed-forward -- share ONE input projection and ONE output projection) and Nivotar
-(:class:`PostNormLayer`: sublayers read the residual stream itself, the norm sits on each sublayer's result).
+output side by side, and -- with a dense feed-forward -- share ONE input projection and ONE output projection), Nivotar
+(:class:`PostNormLayer`: sublayers read the residual stream itself, the norm sits on each sublayer's result) and Tusasun
+(:class:`StreamLayer`: several residual streams that every sublayer reads, mixes and writes through learned vectors).
 """
 
 from __future__ import annotations
@@ -55,10 +64,10 @@ from .distributed.parallel_state import get_tp_world_size
 from .kernels.activations import xielu
 from .kernels.attention import (conv_rope_cache, latent_kv_prep, qk_norm_cache, ragged_attention, rotate_pairs, rotation_table,
                                 rownorm_rope_cache)
-from .kernels.fused_moe import group_router, sparse_glu_experts
-from .kernels.norm_act import (GatedUpdate, SummedUpdate, add_rmsnorm_shift, cast_pair, embed_pair, gated_group_norm, glu_act,
-                               residual_set, softcap_)
-from .kernels.recurrent import conv_act, gated_linear_scan, gated_out_norm, linear_scan, mingru_scan
+from .kernels.fused_moe import group_router, sparse_glu_experts, sparse_square_experts
+from .kernels.norm_act import (GatedUpdate, StreamUpdate, SummedUpdate, add_rmsnorm_shift, cast_pair, embed_pair, gated_group_norm,
+                               glu_act, relu_square, residual_set, softcap_, stream_norm)
+from .kernels.recurrent import (conv_act, delta_scan, gated_linear_scan, gated_out_norm, linear_scan, mingru_scan, rglru_scan)
 from .linear import ReplicatedLinear
 
 
@@ -127,6 +136,7 @@ class StateSpaceSpec:
 @dataclass(frozen=True)
 class MixerSpec:
     kind: str                   # "attention" | "hgrn2" | "latent_attention" | "mingru" | "conv_attention" | "attention_ssd" | "decay_linear" | "gla"
+                                # | "distance_attention" | "channel_delta" | "rglru"
     heads: int = 1
     dim: int = 0                # per-head query / key width (latent attention: the unrotated part)
     vdim: int = 0               # per-head value width
@@ -140,28 +150,34 @@ class MixerSpec:
     window: int = 0             # latent / conv attention: 0 = causal, else the last `window` positions are seen
     keep_first: int = 0         # conv attention: with a window, the sequence's first positions that stay visible
     bias: bool = False          # conv attention: q / k / v projections carry a bias
-    conv_taps: int = 0          # conv attention: taps of the causal convolution over time behind the projections (0: none)
+    conv_taps: int = 0          # conv attention, channel_delta, rglru: taps of the causal convolution over time behind the projections (0: none)
     unit_norm: bool = False     # conv attention: q / k heads divided by their root mean square (no weight) after the rotation
     unit_sink: bool = False     # conv attention: a key of score 0 without a value in every softmax denominator
     value_mix: bool = False     # conv attention: values blended with those of the first layer that says so
     out_gate: bool = False      # latent attention: heads times sigmoid(W_g h) before the output projection
     rotary: RotarySpec | None = None
-    width: int = 0              # mingru: channels of the recurrence
+    width: int = 0              # mingru, rglru: channels of the recurrence
+    blocks: int = 1             # rglru: equal parts of the channels with gate matrices of their own
     ssd: StateSpaceSpec | None = None           # attention_ssd: the state-space branch beside the attention
     branch_scales: tuple = (1.0, 1.0)           # attention_ssd: result = scales[0] * attention + scales[1] * state-space
     decay: tuple = ()           # decay_linear: the fixed decay of every head
     tau: float = 1.0            # gla: decay = sigmoid(.)^(1 / tau)
-    decay_rank: int = 0         # gla: width of the low-rank projection in front of the decay logits
+    decay_rank: int = 0         # gla, channel_delta: width of the low-rank projection in front of the decay logits
+    gate_rank: int = 0          # channel_delta: width of the low-rank projection in front of the output gate
+    softcap: float = 0.0        # distance attention: scaled scores <- cap tanh(scores / cap) (0: none)
+    bias_rows: int = 0          # distance attention: buckets of the distance bias ..
+    bias_max: float = 0.0       # .. the last of which holds every distance from here on
 
 
 @dataclass(frozen=True)
 class MlpSpec:
     kind: str = "dense"         # "dense" | "moe"
     ff: int = 0                 # dense: hidden width; moe: hidden width of one expert
-    act: str = "xielu"          # dense: "xielu" (up / down) | "gelu_tanh" | "clamped" | "silu" (gate / up / down)
+    act: str = "xielu"          # dense: "xielu" (up / down) | "gelu_tanh" | "clamped" | "silu" (gate / up / down); moe: also "relu_square" (up / down)
     limit: float = 0.0          # "clamped": gate <= limit, |up| <= limit
     scoring: str = "sigmoid"    # moe: "sigmoid" (scores over groups) | "softmax_chosen" (largest logits, softmax over them)
                                 # | "softmax_all" (softmax over all outputs, chosen by score + correction)
+                                # | "sigmoid_plain" (sigmoid scores, not renormalised)
     identity: int = 0           # moe, "softmax_all": router outputs beyond `experts` that stand for the input itself
     bias: bool = False          # dense: every projection carries a bias
     experts: int = 0
@@ -203,6 +219,9 @@ class LayeredGeometry:
     logit_scale: float = 1.0    # logits = head(norm(x)) times this
     tied_head: bool = False     # the output head is the embedding table
     post_norm: bool = False     # sublayers read the residual stream itself; each sublayer's RESULT is normed, then added
+    streams: int = 0            # > 0: this many residual streams, mixed by every sublayer; result rows scaled per channel
+    norm_base: float = 0.0      # added to the layers' and the final norm weights (1: weights stored around zero)
+    loop_mix: bool = True       # a pass starts from a projection of [stream | embedding] (+ a vector per pass)
     extra: dict = field(default_factory=dict, compare=False)
 
     @property
@@ -224,6 +243,8 @@ class LayeredGeometry:
         """``shapes``: ``{tensor name: shape}`` of the checkpoint, for sizes that only a tensor's shape gives."""
         if name == "nivotar":
             return _nivotar_geometry(config, name, shapes or {})
+        if name == "tusasun":
+            return _tusasun_geometry(config, name, shapes or {})
         if name == "rukedra":
             return _rukedra_geometry(config, name)
         if name == "fekanex":
@@ -246,13 +267,19 @@ class LayeredGeometry:
             if mlp is not None and mlp.get("kind", "dense") != "dense":
                 raise ValueError(f"unsupported feed-forward kind {mlp.get('kind')!r}; supported: dense")
             layers.append(LayerSpec(spec, ff=int(mlp["ff"]) if mlp is not None else 0))
-        loop = config.get("loop") or {}
-        start, stop, times = int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1))
-        if stop > start and not (0 <= start < stop <= len(layers) and times >= 1):
-            raise ValueError(f"loop {start}..{stop} x {times} does not fit {len(layers)} layers")
+        start, stop, times = _loop_span(config, len(layers))
         return LayeredGeometry(name=name, vocab_size=int(config["vocab"]), width=int(config["width"]),
                                eps=float(config["norm"]["eps"]), layers=tuple(layers), loop_start=start, loop_stop=stop,
-                               loop_times=times if stop > start else 1)
+                               loop_times=times)
+
+
+def _loop_span(config: Mapping, layers: int) -> tuple[int, int, int]:
+    """``(start, stop, times)`` of the layers that run several times in a row (an empty span: none do)."""
+    loop = config.get("loop") or {}
+    start, stop, times = int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1))
+    if stop > start and not (0 <= start < stop <= layers and times >= 1):
+        raise ValueError(f"loop {start}..{stop} x {times} does not fit {layers} layers")
+    return start, stop, times if stop > start else 1
 
 
 def _rukedra_geometry(config: Mapping, name: str) -> LayeredGeometry:
@@ -404,8 +431,74 @@ def _nivotar_geometry(config: Mapping, name: str, shapes: Mapping) -> LayeredGeo
                            layers=tuple(layers), token_shift=False, tied_head=True, post_norm=True)
 
 
+def _tusasun_geometry(config: Mapping, name: str, shapes: Mapping) -> LayeredGeometry:
+    """Tusasun: per layer one of three mixers -- ``rglru`` (real-gated recurrence behind a convolution), ``attention`` (capped
+    scores with a bias per distance bucket), ``channel_delta`` (gated delta rule with a decay per key entry) --, squared-relu
+    experts with a shared one, several residual streams mixed by every sublayer, norm weights stored around zero, a span of
+    layers that runs several times.  Sizes that only a tensor's shape gives (``shapes``): the rows of ``mix.rel``, ``mix.a1``
+    and ``mix.g1``; a configuration built without a checkpoint names them ``mixer.bias_rows`` / ``rank`` / ``gate_rank``."""
+    layers = []
+    for index, entry in enumerate(config["layers"]):
+        m, kind = entry["mixer"], entry["type"]
+
+        def rows_of(leaf, key):
+            shape = shapes.get(f"l{index}.mix.{leaf}")
+            return int(shape[0]) if shape is not None else int(m.get(key) or 0)
+
+        if kind == "rglru":
+            spec = MixerSpec("rglru", width=int(m["width"]), blocks=int(m["blocks"]), conv_taps=int(m["conv"]))
+            if spec.blocks < 1 or spec.width % spec.blocks or spec.conv_taps < 1:
+                raise ValueError(f"layer {index}: {spec.width} channels do not divide into {spec.blocks} parts, or no convolution tap")
+        elif kind == "attention":
+            spec = MixerSpec("distance_attention", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             kv_heads=int(m.get("kv_heads") or m["heads"]), scale=float(m["scale"]), softcap=float(m.get("softcap") or 0.0),
+                             bias_rows=rows_of("rel", "bias_rows"), bias_max=float(m["bias_max"]))
+            if spec.bias_rows < 2 or spec.bias_max <= spec.bias_rows // 2 or spec.softcap < 0:
+                raise ValueError(f"layer {index}: {spec.bias_rows} distance buckets up to {spec.bias_max} (tensor mix.rel; the first half "
+                                 "holds one distance each)")
+        elif kind == "channel_delta":
+            spec = MixerSpec("channel_delta", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             kv_heads=int(m.get("kv_heads") or m["heads"]), conv_taps=int(m["conv"]), decay_rank=rows_of("a1", "rank"),
+                             gate_rank=rows_of("g1", "gate_rank"))
+            if spec.decay_rank < 1 or spec.gate_rank < 1 or spec.conv_taps < 1:
+                raise ValueError(f"layer {index}: the ranks of the decay and gate projections (tensors mix.a1, mix.g1) must be known, "
+                                 "and a convolution has a tap")
+        else:
+            raise ValueError(f"unsupported mixer type {kind!r}; supported: rglru, attention, channel_delta")
+        if kind != "rglru" and spec.heads % spec.kv_heads:
+            raise ValueError(f"layer {index}: {spec.heads} heads do not divide over {spec.kv_heads} key/value heads")
+        mlp = entry.get("mlp")
+        if mlp is None:
+            mspec = None
+        elif mlp.get("kind", "moe") == "moe":
+            r = mlp["router"]
+            mspec = MlpSpec("moe", ff=int(mlp["expert"]["ff"]), act="relu_square", experts=int(r["experts"]), top=int(r["top"]),
+                            scoring="sigmoid_plain", shared_ff=int((mlp.get("shared") or {}).get("ff", 0)))
+            if not 1 <= mspec.top <= mspec.experts:
+                raise ValueError(f"layer {index}: {mspec.top} of {mspec.experts} experts cannot be chosen")
+        else:
+            raise ValueError(f"unsupported feed-forward kind {mlp.get('kind')!r}; supported: moe")
+        layers.append(LayerSpec(spec, ff=mspec.ff if mspec else 0, mlp_kind=mspec.kind if mspec else "dense", mlp=mspec))
+    start, stop, times = _loop_span(config, len(layers))
+    streams = int(config["streams"])
+    if not 1 <= streams <= 32:
+        raise ValueError(f"{streams} residual streams; supported: 1 .. 32")
+    return LayeredGeometry(name=name, vocab_size=int(config["vocab"]), width=int(config["width"]), eps=float(config["norm"]["eps"]),
+                           layers=tuple(layers), loop_start=start, loop_stop=stop, loop_times=times, token_shift=False, loop_mix=False,
+                           streams=streams, norm_base=1.0)
+
+
 def _linear(inp: int, out: int) -> ReplicatedLinear:
     return ReplicatedLinear(inp, out)
+
+
+def _padded_linear(inp: int, out: int, used_rows: int) -> ReplicatedLinear:
+    """A projection fused from members that start on 16-byte borders: ``out`` rows of which the members fill ``used_rows``, the rest
+    are zeros that no checkpoint tensor fills."""
+    lin = ReplicatedLinear(inp, out)
+    lin.weight.data.zero_()
+    lin.weight.ll_unfilled = (out - used_rows) * inp
+    return lin
 
 
 def _vector(n: int) -> nn.Parameter:
@@ -851,9 +944,162 @@ class CorrectedSoftmaxMoE(nn.Module):
         return y, None, (h if s.identity else None), own
 
 
+def distance_buckets(rows: int, far: float) -> list[int]:
+    """Bucket of the distances 0, 1, .. among ``rows``: one per distance in the first half, then logarithmic up to ``far``; every
+    distance beyond the list is in its last bucket."""
+    half, out = rows // 2, []
+    while not out or out[-1] < rows - 1:
+        n = len(out)
+        out.append(n if n < half else min(rows - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (rows - half))))
+    return out
+
+
+class BiasedDistanceAttention(nn.Module):
+    """``q | k | v`` in one biased projection, then per-head norm + cache write (one launch), attention over the paged cache with
+    capped scores and a learned bias per head and distance bucket (one launch), biased output projection."""
+
+    def __init__(self, width: int, spec: MixerSpec, eps: float):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        self.in_proj = ReplicatedLinear(width, (spec.heads + spec.kv_heads) * spec.dim + spec.kv_heads * spec.vdim, bias=True)
+        self.o_proj = ReplicatedLinear(spec.heads * spec.vdim, width, bias=True)
+        self.q_norm_weight = _vector(spec.dim)
+        self.k_norm_weight = _vector(spec.dim)
+        self.bias_table = nn.Parameter(torch.zeros(spec.bias_rows, spec.heads, dtype=torch.float16), requires_grad=False)
+        self._by_distance = None   # fp32 [heads, distances], spread from the buckets at the first step
+
+    def invalidate_derived(self) -> None:
+        self._by_distance = None
+
+    def cache_run(self) -> dict:
+        return {"kind": "attention", "kv_heads": self.spec.kv_heads, "dk": self.spec.dim, "dv": self.spec.vdim}
+
+    def forward(self, h, step, cache, run: int, token_table):
+        s = self.spec
+        if self._by_distance is None or self._by_distance.device != h.device:
+            index = torch.tensor(distance_buckets(s.bias_rows, s.bias_max), device=h.device)
+            self._by_distance = self.bias_table.float()[index].t().contiguous()
+        k_cache, v_cache = cache.kv_buffer[run]
+        q = qk_norm_cache(self.in_proj(h), s.heads, s.kv_heads, s.dim, s.vdim, self.q_norm_weight, self.k_norm_weight, self.eps, 0.0, 1,
+                          step, k_cache, v_cache)
+        return self.o_proj(ragged_attention(q, k_cache, v_cache, s.scale, step, token_table, cap=s.softcap, dist_bias=self._by_distance))
+
+
+def _aligned(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+class ChannelDeltaMixer(nn.Module):
+    """``q | k | v | a1 | g1 | b`` in one projection (members on 16-byte borders); q, k, v through one short convolution and silu; the
+    decay logits and the output gate's logits from ``a1 | g1`` in one block-diagonal projection; gated delta rule over the fp32
+    state slots (unit q / k heads, decay per key entry, a step size per head); every head RMS-normed with one shared weight, times
+    the sigmoid of its gate; output projection."""
+
+    unit_eps = 1e-6   # inside the root of the q / k unit norms
+
+    def __init__(self, width: int, spec: MixerSpec, eps: float):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        s = spec
+        self.qk, self.gk, self.v = s.kv_heads * s.dim, s.heads * s.dim, s.heads * s.vdim
+        self.channels = 2 * self.qk + self.v
+        self.low_off = _aligned(self.channels)
+        self.beta_off = _aligned(self.low_off + s.decay_rank + s.gate_rank)
+        self.in_proj = _padded_linear(width, _aligned(self.beta_off + s.heads), self.channels + s.decay_rank + s.gate_rank + s.heads)
+        self.conv_weight = nn.Parameter(torch.zeros(self.channels, s.conv_taps, dtype=torch.float16), requires_grad=False)
+        # [decay logits | gate logits] = diag(W_a2, W_g2) [a1 | g1]: the two off-diagonal parts stay zero
+        self.gate_off = _aligned(self.gk)
+        self.low_proj = ReplicatedLinear(s.decay_rank + s.gate_rank, self.gate_off + _aligned(self.v))
+        self.low_proj.weight.data.zero_()
+        self.low_proj.weight.ll_unfilled = self.low_proj.weight.numel() - self.gk * s.decay_rank - self.v * s.gate_rank
+        self.dt_bias, self.a_log = _vector(self.gk), _vector(s.heads)
+        self.out_norm_weight = _vector(s.vdim)
+        self.o_proj = _linear(self.v, width)
+
+    def cache_run(self) -> dict:
+        s = self.spec
+        return {"kind": "recurrent", "heads": s.heads, "dk": s.dim, "dv": s.vdim, "conv_taps": s.conv_taps, "conv_channels": self.channels}
+
+    def forward(self, h, step, cache, run: int, token_table):
+        s, qk = self.spec, self.qk
+        rows = self.in_proj(h)
+        qkv = conv_act(rows[:, :self.channels], self.conv_weight, None, step, cache.conv[run])
+        low = self.low_proj(rows[:, self.low_off:self.low_off + s.decay_rank + s.gate_rank].contiguous())
+        o = delta_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], s.heads, s.dim, s.vdim, step, cache.recurrent[run],
+                       gate=low[:, :self.gk], dt_bias=self.dt_bias, a_log=self.a_log, beta=rows[:, self.beta_off:self.beta_off + s.heads],
+                       qk_heads=s.kv_heads, q_scale=s.dim ** -0.5, unit_eps=self.unit_eps)
+        return self.o_proj(gated_out_norm(o, self.out_norm_weight, self.eps, parts=s.heads,
+                                          gate=low[:, self.gate_off:self.gate_off + self.v], gate_kind="sigmoid"))
+
+
+class RealGatedLRU(nn.Module):
+    """``x | y`` in one biased projection; ``x`` through a short convolution (with bias, no activation); both gates of the recurrence as
+    one batched product over the diagonal blocks; gates, recurrence and the gelu-gated read-out over the fp32 state slots; output
+    projection."""
+
+    def __init__(self, width: int, spec: MixerSpec, eps: float):
+        super().__init__()
+        self.spec = spec
+        w, bs = spec.width, spec.width // spec.blocks
+        self.y_off = _aligned(w)
+        self.in_proj = ReplicatedLinear(width, self.y_off + _aligned(w), bias=True)
+        for p in (self.in_proj.weight, self.in_proj.bias):
+            p.data.zero_()
+            p.ll_unfilled = (p.shape[0] - 2 * w) * (p.numel() // p.shape[0])
+        self.conv_weight = nn.Parameter(torch.zeros(w, spec.conv_taps, dtype=torch.float16), requires_grad=False)
+        self.conv_bias = _vector(w)
+        # per block [in][r | i]: the right operand of the batched product is contiguous
+        self.gate_weight = nn.Parameter(torch.zeros(spec.blocks, bs, 2 * bs, dtype=torch.float16), requires_grad=False)
+        self.r_bias, self.i_bias, self.lam = _vector(w), _vector(w), _vector(w)
+        self.o_proj = _linear(w, width)
+
+    def cache_run(self) -> dict:
+        w = self.spec.width
+        return {"kind": "recurrent", "heads": 1, "dk": 1, "dv": w, "conv_taps": self.spec.conv_taps, "conv_channels": w}
+
+    def forward(self, h, step, cache, run: int, token_table):
+        w, blocks = self.spec.width, self.spec.blocks
+        bs, n = w // blocks, h.shape[0]
+        rows = self.in_proj(h)
+        u = conv_act(rows[:, :w], self.conv_weight, self.conv_bias, step, cache.conv[run], act=None)
+        gates = torch.empty(n, blocks, 2 * bs, dtype=h.dtype, device=h.device)
+        torch.bmm(u.view(n, blocks, bs).transpose(0, 1), self.gate_weight, out=gates.transpose(0, 1))
+        o = rglru_scan(u, gates.view(n, blocks, 2, bs), self.r_bias, self.i_bias, self.lam, rows[:, self.y_off:self.y_off + w], step,
+                       cache.recurrent[run].view(-1, w))
+        return self.o_proj(o)
+
+
+class SquareMoE(nn.Module):
+    """Sigmoid router (fp32) whose chosen scores multiply the experts' INPUTS, not renormalised; experts ``down(relu(up h)^2)`` without
+    biases as grouped products over slots sorted by expert; a shared expert of the same form whose result is scaled per token by
+    ``sigmoid(w_sg . h)``.  The slots' rows are NOT summed here: they ride, with the shared row and its scale, into the launch that
+    mixes the streams."""
+
+    def __init__(self, width: int, spec: MlpSpec):
+        super().__init__()
+        self.spec = spec
+        self.router_weight = nn.Parameter(torch.zeros(spec.experts, width, dtype=torch.float16), requires_grad=False)
+        self.up_weight = nn.Parameter(torch.zeros(spec.experts, spec.ff, width, dtype=torch.float16), requires_grad=False)
+        self.down_weight = nn.Parameter(torch.zeros(spec.experts, width, spec.ff, dtype=torch.float16), requires_grad=False)
+        if spec.shared_ff:
+            self.shared_up_proj = _linear(width, spec.shared_ff)
+            self.shared_down_proj = _linear(spec.shared_ff, width)
+            self.shared_scale_weight = nn.Parameter(torch.zeros(1, width, dtype=torch.float16), requires_grad=False)
+
+    def forward(self, h):
+        """``(slots' rows [n, top, width], shared row or None, its scale or None)``."""
+        s = self.spec
+        ids, weights, scale = group_router(h, self.router_weight, s.top, scoring=s.scoring,
+                                           extra_weight=self.shared_scale_weight if s.shared_ff else None)
+        y = sparse_square_experts(h, self.up_weight, self.down_weight, ids, weights)
+        shared = self.shared_down_proj(relu_square(self.shared_up_proj(h), s.shared_ff)) if s.shared_ff else None
+        return y, shared, scale
+
+
 MIXERS = {"attention": SinkAttention, "hgrn2": GatedLinearMixer, "latent_attention": LatentAttention, "mingru": MinGRU,
           "conv_attention": ConvRotaryAttention, "attention_ssd": WindowAttentionSSD, "decay_linear": DecayLinearAttention,
-          "gla": GatedLinearAttention}
+          "gla": GatedLinearAttention, "distance_attention": BiasedDistanceAttention, "channel_delta": ChannelDeltaMixer,
+          "rglru": RealGatedLRU}
 
 
 class MixerLayer(nn.Module):
@@ -967,6 +1213,48 @@ class PostNormLayer(nn.Module):
         return x, pending
 
 
+class StreamMix(nn.Module):
+    """What one sublayer does to the residual streams: how its input is gathered, how the streams are mixed, how much of its result
+    (scaled per channel) every stream receives."""
+
+    def __init__(self, streams: int, width: int):
+        super().__init__()
+        self.gather, self.out = _vector(streams), _vector(streams)
+        self.mix = nn.Parameter(torch.zeros(streams, streams, dtype=torch.float16), requires_grad=False)   # [from, to]
+        self.scale = _vector(width)
+
+    def update(self, y, shared=None, shared_scale=None) -> StreamUpdate:
+        return StreamUpdate(y, self.scale, self.mix, self.out, shared, shared_scale)
+
+
+class StreamLayer(nn.Module):
+    """``u = sum_s in_s x_s``, ``x_t <- sum_s mix[s, t] x_s + out_t (scale * f(norm(u)))`` for the mixer and then for the feed-forward,
+    over several residual streams.  A sublayer's result is carried as a :class:`StreamUpdate` into the launch that opens the next
+    sublayer: result sum, scale, mixing, gathering and norm are one launch."""
+
+    def __init__(self, geo: LayeredGeometry, spec: LayerSpec):
+        super().__init__()
+        self.eps, self.base, self.streams = geo.eps, geo.norm_base, geo.streams
+        w, m = geo.width, spec.mixer
+        self.norm1_weight = _vector(w)
+        self.mix1 = StreamMix(geo.streams, w)
+        self.mixer = MIXERS[m.kind](w, m, geo.eps)
+        self.mlp = None
+        if spec.mlp is not None:
+            self.norm2_weight = _vector(w)
+            self.mix2 = StreamMix(geo.streams, w)
+            self.mlp = SquareMoE(w, spec.mlp)
+
+    def forward(self, x, pending, step, cache, run: int, token_table):
+        """``(x, pending)``: the fp32 streams and the update still to enter them.  Returns the same pair."""
+        h, x = stream_norm(x, pending, self.streams, self.mix1.gather, self.norm1_weight, self.eps, self.base)
+        pending = self.mix1.update(self.mixer(h, step, cache, run, token_table))
+        if self.mlp is not None:
+            h, x = stream_norm(x, pending, self.streams, self.mix2.gather, self.norm2_weight, self.eps, self.base)
+            pending = self.mix2.update(*self.mlp(h))
+        return x, pending
+
+
 # ------------------------------------------------------------------------------------- #
 # the model
 # ------------------------------------------------------------------------------------- #
@@ -980,11 +1268,12 @@ class LayeredLM(nn.Module):
         self.geo = geo
         self.embed_tokens = nn.Embedding(geo.vocab_size, geo.width, dtype=torch.float16)
         self.embed_tokens.weight.requires_grad_(False)
-        make = SandwichLayer if geo.sandwich else ParallelLayer if geo.parallel else PostNormLayer if geo.post_norm else MixerLayer
+        make = (SandwichLayer if geo.sandwich else ParallelLayer if geo.parallel else PostNormLayer if geo.post_norm
+                else StreamLayer if geo.streams else MixerLayer)
         # a layer that borrows weights IS the other layer's module (which may come later in the stack); its cache run stays its own
         built = [make(geo, spec) if spec.weights_of is None else None for spec in geo.layers]
         self.layers = nn.ModuleList(built[i] if spec.weights_of is None else built[spec.weights_of] for i, spec in enumerate(geo.layers))
-        if geo.looped:
+        if geo.looped and geo.loop_mix:
             self.loop_in = _linear(2 * geo.width, geo.width)
             self.loop_step = nn.Parameter(torch.zeros(geo.loop_times, geo.width, dtype=torch.float16), requires_grad=False)
         self.norm_weight = _vector(geo.width)
@@ -1022,9 +1311,10 @@ class LayeredLM(nn.Module):
                             self.geo.pair_mul_prev, self.geo.pair_mul_cur, step, cache.prev_token)
         else:
             x0 = residual_set(F.embedding(token_ids, self.embed_tokens.weight))
-        x, delta = (x0.clone() if self.geo.looped else x0), None  # (layers update the residual in place; x0 is read again)
+        loop_mix = self.geo.looped and self.geo.loop_mix
+        x, delta = (x0.clone() if loop_mix else x0), None  # (layers update the residual in place; x0 is read again)
         for run, (index, pass_no, first) in enumerate(self.run_order):
-            if first:
+            if first and loop_mix:
                 y = self.loop_in(cast_pair(x, x0, self.dtype, a_delta=delta))
                 x, delta = residual_set(y, self.loop_step[pass_no]), None
             x, delta = self.layers[index](x, delta, step, cache, run, token_table)
@@ -1033,6 +1323,8 @@ class LayeredLM(nn.Module):
                     seen = x.clone()
                     gated_group_norm(seen, delta, None, self.geo.eps, self.geo.norm_groups)
                     collect_layers.append(seen)
+                elif self.geo.streams:
+                    collect_layers.append(stream_norm(x.clone(), delta, self.geo.streams, None, None, self.geo.eps)[1].sum(1))
                 elif isinstance(delta, SummedUpdate):
                     collect_layers.append(x + delta.total())
                 else:
@@ -1043,6 +1335,9 @@ class LayeredLM(nn.Module):
         if self.geo.sandwich or self.geo.post_norm:
             h = gated_group_norm(x, delta.rows(logits_rows) if delta is not None else None, self.norm_weight, self.geo.eps,
                                  self.geo.norm_groups)
+        elif self.geo.streams:
+            h, _ = stream_norm(x, delta.rows(logits_rows) if delta is not None else None, self.geo.streams, None, self.norm_weight,
+                               self.geo.eps, self.geo.norm_base)
         else:
             if isinstance(delta, SummedUpdate):
                 delta = delta.rows(logits_rows)
@@ -1070,16 +1365,28 @@ class LayeredLM(nn.Module):
 
         for name, p in self.named_parameters():
             leaf = name.rsplit(".", 1)[-1]
-            if name.endswith("proj.weight") or name.endswith("lm_head.weight"):
+            if self.geo.norm_base and leaf in ("norm1_weight", "norm2_weight", "norm_weight"):
+                fill(p, std=0.1, mean=1.0 - self.geo.norm_base)
+            elif leaf in ("gather", "out"):         # (streams: the plain residual sum, disturbed a little)
+                fill(p, std=0.1, mean=1.0 if leaf == "out" else 1.0 / self.geo.streams)
+            elif leaf == "mix":
+                fill(p, std=0.1)
+                p.data.add_(torch.eye(self.geo.streams, dtype=p.dtype, device=p.device))
+            elif leaf in ("scale", "lam"):
+                fill(p, lo=0.2, hi=0.8)
+            elif name.endswith("proj.weight") or name.endswith("lm_head.weight"):
                 fill(p, std=1.0 / (p.shape[1] ** 0.5))
             elif name in ("embed_tokens.weight", "pair_table"):
                 fill(p, std=1.0)
             elif leaf in ("norm1_weight", "norm2_weight", "norm_weight", "q_norm_weight", "k_norm_weight", "out_norm_weight",
                           "norm1b_weight", "norm2b_weight", "kv_norm_weight", "ssd_norm_weight"):
                 fill(p, std=0.1, mean=1.0)
-            elif leaf in ("uk_weight", "uv_weight", "router_weight", "gate_up_weight", "down_weight", "shared_scale_weight"):
+            elif leaf in ("uk_weight", "uv_weight", "router_weight", "gate_up_weight", "down_weight", "up_weight", "shared_scale_weight"):
                 fill(p, std=1.0 / (p.shape[-1] ** 0.5))
-            elif leaf in ("rg1_bias", "rg2_bias", "z_bias", "x_bias", "qkv_bias", "conv_bias", "down_bias", "decay_bias", "dt_bias") \
+            elif leaf == "gate_weight":             # (stored [part, in, out])
+                fill(p, std=1.0 / (p.shape[1] ** 0.5))
+            elif leaf in ("rg1_bias", "rg2_bias", "z_bias", "x_bias", "qkv_bias", "conv_bias", "down_bias", "decay_bias", "dt_bias", "r_bias", "i_bias",
+                          "bias_table") \
                     or name.endswith("proj.bias"):
                 fill(p, std=0.5)
             elif leaf in ("a_log", "skip"):

@@ -43,11 +43,16 @@ class Region:
     parts: int = 2
     rows: tuple[int, int] | None = None   # (first row, count): one member of a projection fused from UNEQUAL members
     cols: tuple[int, int] | None = None   # (first column, count): one member of a projection fused along its INPUT
+    transposed_cols: tuple[int, int] | None = None   # (first column, count) of a stack of matrices kept transposed ([.., in, out])
     entry: int | None = None    # one entry of a vector, filled by a checkpoint tensor without dimensions
 
     def __call__(self, param: torch.Tensor) -> torch.Tensor:
         view = param if self.expert is None else param[self.expert]
+        if self.transposed_cols is not None:
+            return view.narrow(-1, self.transposed_cols[0], self.transposed_cols[1]).transpose(-1, -2)
         if self.cols is not None:
+            if self.rows is not None:   # one block of a block-diagonal projection
+                view = view.narrow(0, self.rows[0], self.rows[1])
             return view.narrow(1, self.cols[0], self.cols[1])
         if self.entry is not None:
             return view[self.entry]
@@ -381,6 +386,8 @@ def invalidate_derived_layouts(model: nn.Module) -> None:
         if hasattr(p_.data, "_ll_prepacked"):
             delattr(p_.data, "_ll_prepacked")
     for mod in model.modules():
+        if hasattr(mod, "invalidate_derived"):
+            mod.invalidate_derived()
         for attr in ("_w4_prepacked", "_w4_packed", "_tp_fused_cache"):
             if hasattr(mod, attr):
                 delattr(mod, attr)
@@ -391,7 +398,9 @@ def invalidate_derived_layouts(model: nn.Module) -> None:
 
 def _verify_coverage(params: Mapping[str, nn.Parameter], filled: Mapping[str, int]) -> None:
     never = sorted(n for n, c in filled.items() if c == 0)
-    wrong = sorted(f"{n} ({c} of {params[n].numel()} elements)" for n, c in filled.items() if 0 < c != params[n].numel())
+    # (a parameter may hold zeros that no checkpoint tensor fills: padding between the members of a fused projection)
+    expected = {n: params[n].numel() - int(getattr(params[n], "ll_unfilled", 0)) for n in filled}
+    wrong = sorted(f"{n} ({c} of {expected[n]} elements)" for n, c in filled.items() if 0 < c != expected[n])
     if not never and not wrong:
         return
     problems = []
@@ -773,6 +782,75 @@ def _nivotar_translator(geo) -> Translator:
     return translate
 
 
+def _tusasun_translator(geo, layers) -> Translator:
+    """Tensor names of a Tusasun checkpoint -> parameters of :class:`lite_llama_amd.model_layers.LayeredLM` built from
+    :class:`StreamLayer`.  Everything that reads a mixer's input lands in its row range of the mixer's ONE input projection
+    (``q | k | v``, biased; ``q | k | v | a1 | g1 | b``; ``x | y``, biased -- members on 16-byte borders); ``a2`` / ``g2`` are the two
+    diagonal blocks of one projection; ``ra`` / ``ri`` are kept transposed side by side; experts ``mlp.e<k>.*`` in the stacked expert
+    tensors; ``hc<n>.*`` and ``ls<n>`` in the layer's two stream mixes.  ``layers``: the model's layers (their fused projections know
+    where their members lie)."""
+    fixed = {"embed": "embed_tokens.weight", "final.norm": "norm_weight", "head": "lm_head.weight"}
+    plain = {"norm1": "norm1_weight", "norm2": "norm2_weight", "mix.o": "mixer.o_proj.weight", "mix.o.b": "mixer.o_proj.bias",
+             "mix.q.norm": "mixer.q_norm_weight", "mix.k.norm": "mixer.k_norm_weight", "mix.rel": "mixer.bias_table",
+             "mix.A_log": "mixer.a_log", "mix.dt_bias": "mixer.dt_bias", "mix.norm": "mixer.out_norm_weight", "mix.lam": "mixer.lam",
+             "mix.conv": "mixer.conv_weight", "mix.conv.b": "mixer.conv_bias", "mlp.router": "mlp.router_weight",
+             "mlp.shared.up": "mlp.shared_up_proj.weight", "mlp.shared.down": "mlp.shared_down_proj.weight",
+             "mlp.shared.sg": "mlp.shared_scale_weight"}
+    for n in (1, 2):
+        plain.update({f"ls{n}": f"mix{n}.scale", f"hc{n}.in": f"mix{n}.gather", f"hc{n}.out": f"mix{n}.out", f"hc{n}.mix": f"mix{n}.mix"})
+    expert_leaf = re.compile(r"^mlp\.e(\d+)\.(up|down)$")
+
+    def fused(layer, spec):
+        """``{checkpoint leaf: (parameter, Region)}`` of one layer."""
+        m, out = spec.mixer, {}
+
+        def rows(param, members):
+            for leaf, first, count in members:
+                out[leaf] = (param, Region(rows=(first, count)))
+
+        if m.kind == "distance_attention":
+            q, k, v = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
+            members = (("mix.q", 0, q), ("mix.k", q, k), ("mix.v", q + k, v))
+            rows("mixer.in_proj.weight", members)
+            rows("mixer.in_proj.bias", tuple((leaf + ".b", first, count) for leaf, first, count in members))
+        elif m.kind == "channel_delta":
+            x = layer.mixer
+            members = (("mix.q", 0, x.qk), ("mix.k", x.qk, x.qk), ("mix.v", 2 * x.qk, x.v))
+            rows("mixer.in_proj.weight", members + (("mix.a1", x.low_off, m.decay_rank), ("mix.g1", x.low_off + m.decay_rank, m.gate_rank),
+                                                    ("mix.b", x.beta_off, m.heads)))
+            rows("mixer.conv_weight", tuple((leaf + ".conv", first, count) for leaf, first, count in members))
+            out["mix.a2"] = ("mixer.low_proj.weight", Region(rows=(0, x.gk), cols=(0, m.decay_rank)))
+            out["mix.g2"] = ("mixer.low_proj.weight", Region(rows=(x.gate_off, x.v), cols=(m.decay_rank, m.gate_rank)))
+        else:
+            w, bs, y = m.width, m.width // m.blocks, layer.mixer.y_off
+            rows("mixer.in_proj.weight", (("mix.x", 0, w), ("mix.y", y, w)))
+            rows("mixer.in_proj.bias", (("mix.x.b", 0, w), ("mix.y.b", y, w)))
+            out["mix.ra"] = ("mixer.gate_weight", Region(transposed_cols=(0, bs)))
+            out["mix.ri"] = ("mixer.gate_weight", Region(transposed_cols=(bs, bs)))
+            out["mix.ra.b"] = ("mixer.r_bias", lambda p: p.view(m.blocks, bs))
+            out["mix.ri.b"] = ("mixer.i_bias", lambda p: p.view(m.blocks, bs))
+        return out
+
+    members = [fused(layer, spec) for layer, spec in zip(layers, geo.layers)]
+
+    def translate(key: str) -> Target:
+        if key in fixed:
+            return fixed[key], whole
+        m = re.match(r"^l(\d+)\.(.+)$", key)
+        if m is None or int(m.group(1)) >= len(geo.layers):
+            return key, whole  # unknown: load_weights reports it
+        index, leaf = int(m.group(1)), m.group(2)
+        if leaf in members[index]:
+            name, region = members[index][leaf]
+            return f"layers.{index}.{name}", region
+        e = expert_leaf.match(leaf)
+        if e is not None:
+            return f"layers.{index}.mlp.{e.group(2)}_weight", expert(int(e.group(1)))
+        return f"layers.{index}.{plain.get(leaf, leaf)}", whole
+
+    return translate
+
+
 def tensor_shapes(checkpoints_dir: str | Path) -> dict[str, tuple[int, ...]]:
     """``{tensor name: shape}`` of a directory's safetensors files (headers only: no tensor is read)."""
     from safetensors import safe_open
@@ -791,17 +869,19 @@ def _load_layered(config: Mapping, checkpoints_dir, device, dtype=None, **_):
     from .model_layers import LayeredGeometry, LayeredLM
 
     family = model_family(config)
-    geo = LayeredGeometry.from_config(config, name=family, shapes=tensor_shapes(checkpoints_dir) if family == "nivotar" else None)
+    geo = LayeredGeometry.from_config(config, name=family,
+                                      shapes=tensor_shapes(checkpoints_dir) if family in ("nivotar", "tusasun") else None)
     model = LayeredLM(geo, dtype=dtype or torch.bfloat16).to(device)
     translator = (_rukedra_translator(geo) if geo.sandwich else _fekanex_translator(geo) if geo.parallel
-                  else _nivotar_translator(geo) if geo.post_norm else _layered_translator(geo))
+                  else _nivotar_translator(geo) if geo.post_norm else _tusasun_translator(geo, model.layers) if geo.streams
+                  else _layered_translator(geo))
     with torch.no_grad():
         load_weights(model, hf_weights_iterator(checkpoints_dir, device), translator)
     return model.eval()
 
 
 MODEL_FAMILIES: dict[str, Callable] = {"rakevik": _load_layered, "rukedra": _load_layered, "fekanex": _load_layered,
-                                       "nivotar": _load_layered}
+                                       "nivotar": _load_layered, "tusasun": _load_layered}
 
 
 def load_pretrained(checkpoints_dir: str | Path, *, device: str | torch.device = "cuda", quantization: str | None = None,
