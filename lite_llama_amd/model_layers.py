@@ -598,6 +598,10 @@ class LatentAttention(nn.Module):
         self._freq_values, self.amp = s.rotary.table()
         self.pairs = len(self._freq_values)
         self._freq = None   # fp32 on the device of the first step (not a buffer: a module-wide cast must not touch the angles)
+        self._uv_by_rank = None   # uv_weight as [heads, rank, vdim], made at the first step: batched products take a contiguous right operand
+
+    def invalidate_derived(self) -> None:
+        self._uv_by_rank = None
 
     def cache_run(self) -> dict:
         return {"kind": "latent", "rank": self.spec.kv_rank, "rot": self.spec.rot_dim}
@@ -634,8 +638,9 @@ class LatentAttention(nn.Module):
         rotate_pairs(q, s.dim, s.rot_dim, self._freq, self.pairs, self.amp, step, qa, s.kv_rank)
         o_lat = ragged_attention(qa, k_cache, v_cache, s.scale, step, token_table, window=s.window)     # [n, heads * rank]
         o = torch.empty(n, s.heads, s.vdim, dtype=q.dtype, device=q.device)
-        torch.bmm(o_lat.view(n, s.heads, s.kv_rank).transpose(0, 1), self.uv_weight.view(s.heads, s.vdim, s.kv_rank).transpose(1, 2),
-                  out=o.transpose(0, 1))
+        if self._uv_by_rank is None or self._uv_by_rank.device != q.device:
+            self._uv_by_rank = self.uv_weight.view(s.heads, s.vdim, s.kv_rank).transpose(1, 2).contiguous()
+        torch.bmm(o_lat.view(n, s.heads, s.kv_rank).transpose(0, 1), self._uv_by_rank, out=o.transpose(0, 1))
         return o.view(n, s.heads * s.vdim)
 
     def _expanded(self, q, cache_rows, step):
