@@ -113,6 +113,13 @@ def parse():
                          "(benchmarks/nivotar_bench.py); --layered-dtype picks the dtype")
     ap.add_argument("--nivotar-sizes", default="compact,wide", help="which size points of benchmarks/nivotar_bench.py::SIZES to run")
     ap.add_argument("--nivotar-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
+    ap.add_argument("--tusasun", action="store_true",
+                    help="instead of the headline: prefill / decode throughput and per-kernel roofline fractions of the Tusasun design "
+                         "(gated delta rule, real-gated recurrence, capped attention with a bias per distance, squared-relu experts, "
+                         "mixed residual streams) beside the closest model of the layered family (benchmarks/tusasun_bench.py); "
+                         "--layered-dtype picks the dtype")
+    ap.add_argument("--tusasun-sizes", default="compact,wide", help="which size points of benchmarks/tusasun_bench.py::SIZES to run")
+    ap.add_argument("--tusasun-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
     ap.add_argument("--rukedra-sizes", default="compact,wide", help="which size points of benchmarks/rukedra_bench.py::SIZES to run")
     ap.add_argument("--rukedra-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
     ap.add_argument("--no-reference-order", action="store_true",
@@ -948,6 +955,11 @@ def main():
         from benchmarks.rukedra_bench import run as rukedra_run
 
         print(json.dumps(rukedra_run(args.layered_dtype, sizes=tuple(args.rukedra_sizes.split(",")), kernels=not args.rukedra_model_only)))
+        return
+    if args.tusasun:
+        from benchmarks.tusasun_bench import run as tusasun_run
+
+        print(json.dumps(tusasun_run(args.layered_dtype, sizes=tuple(args.tusasun_sizes.split(",")), kernels=not args.tusasun_model_only)))
         return
     if args.nivotar:
         from benchmarks.nivotar_bench import run as nivotar_run

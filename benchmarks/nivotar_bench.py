@@ -161,12 +161,12 @@ def _geometries(width, heads, kv_heads, dim, vdim, rot, window, ssd_heads, ssd_v
     return new, old
 
 
-def model_points(dev, dtype, geos, prefill=(8, 512), decode=(32, 1024), steps=16):
+def model_points(dev, dtype, geos, prefill=(8, 512), decode=(32, 1024), steps=16, labels=("nivotar", "rakevik")):
     from lite_llama_amd.executor.ragged import RaggedRunner
     from lite_llama_amd.model_layers import LayeredLM
 
     res = {}
-    for label, geo in zip(("nivotar", "rakevik"), geos):
+    for label, geo in zip(labels, geos):
         vocab = geo.vocab_size
         model = LayeredLM(geo, dtype=dtype).init_synthetic(0, dev)
         g = torch.Generator().manual_seed(5)
