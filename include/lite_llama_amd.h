@@ -771,15 +771,15 @@ int ll_rownorm_rope_cache(const void* rows, int64_t ld, const void* q_w, const v
  * raw key / query head per heads / qk_rep value heads; a head is divided by sqrt(sum of squares + unit_eps), q also times q_scale.
  * g = exp(-exp(a_log[h]) softplus(gate[t][h dk + i] + dt_bias[h dk + i])) per key entry, beta = sigmoid(beta[t][h]).  o: fp32
  * [n, heads dv].  A run that starts at position 0 starts from zeros.  scratch (fp32, 16-byte aligned, ll_delta_scan_scratch_floats
- * floats, or NULL): decays and per-token scalars are evaluated once, ahead of the walk (same values).  longest_run: most tokens a
- * sequence of the step brings (0: unknown); sizes the staging buffers only.  dk <= 256. */
+ * floats, or NULL): decays and per-token scalars are evaluated once, ahead of the walk (same values; the form for runs of several
+ * tokens).  dk <= 256; state 16-byte aligned. */
 int ll_delta_scan_supported(int64_t dk, int64_t dv);
 int64_t ll_delta_scan_scratch_floats(int64_t n, int64_t heads, int64_t dk);
 int ll_delta_scan(const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, int64_t heads,
                   int64_t dk, int64_t dv, int64_t qk_rep, float q_scale, float unit_eps, const void* gate, int64_t gate_ld,
                   const void* dt_bias, const void* a_log, const void* beta, int64_t beta_ld, float* o, int64_t batch,
                   const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, float* state,
-                  float* scratch, int64_t n, int64_t longest_run, int dtype, void* stream);
+                  float* scratch, int64_t n, int dtype, void* stream);
 
 /* ---- several mixed residual streams (csrc/stream_norm.hip) --------------------------------------------------------------------
  * With y: d = (sum of `parts` rows y[t][p][:] + shared_scale[t] * shared[t][:]) * scale (shared, scale may be NULL) and

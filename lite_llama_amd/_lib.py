@@ -144,7 +144,7 @@ SIGNATURES = {
     "ll_rglru_scan": [P, L, P, L, P, P, P, P, L, P, L, L, L, L, P, P, P, P, L, P, I, P],
     "ll_delta_scan_supported": [L, L],
     "ll_delta_scan_scratch_floats": [L, L, L],
-    "ll_delta_scan": [P, L, P, L, P, L, L, L, L, L, F, F, P, L, P, P, P, L, P, L, P, P, P, P, P, L, L, I, P],
+    "ll_delta_scan": [P, L, P, L, P, L, L, L, L, L, F, F, P, L, P, P, P, L, P, L, P, P, P, P, P, L, I, P],
     "ll_stream_norm": [P, L, L, P, P, L, P, P, P, P, P, P, P, F, F, P, L, L, L, I, P],
 }
 

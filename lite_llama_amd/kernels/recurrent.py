@@ -153,7 +153,7 @@ def delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: int, dk
                                   float(q_scale), float(unit_eps), gate.data_ptr(), ld(gate), dt_bias.data_ptr(), a_log.data_ptr(),
                                   beta.data_ptr(), ld(beta), o.data_ptr(), step.num_seqs, step.seq_start.data_ptr(),
                                   step.seq_first_pos.data_ptr(), step.seq_slot.data_ptr(), state.data_ptr(), L.ptr(scratch), n,
-                                  int(step.longest_run), L.dtype_code(st), L.stream_ptr()), "delta_scan")
+                                  L.dtype_code(st), L.stream_ptr()), "delta_scan")
     return o
 
 
