@@ -1029,7 +1029,7 @@ class ChannelDeltaMixer(nn.Module):
         s, qk = self.spec, self.qk
         rows = self.in_proj(h)
         qkv = conv_act(rows[:, :self.channels], self.conv_weight, None, step, cache.conv[run])
-        low = self.low_proj(rows[:, self.low_off:self.low_off + s.decay_rank + s.gate_rank].contiguous())
+        low = self.low_proj(rows[:, self.low_off:self.low_off + s.decay_rank + s.gate_rank])
         o = delta_scan(qkv[:, :qk], qkv[:, qk:2 * qk], qkv[:, 2 * qk:], s.heads, s.dim, s.vdim, step, cache.recurrent[run],
                        gate=low[:, :self.gk], dt_bias=self.dt_bias, a_log=self.a_log, beta=rows[:, self.beta_off:self.beta_off + s.heads],
                        qk_heads=s.kv_heads, q_scale=s.dim ** -0.5, unit_eps=self.unit_eps)
