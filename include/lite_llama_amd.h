@@ -609,12 +609,13 @@ int ll_qk_norm_cache(const void* qkv, int64_t ld, const void* q_w, const void* k
  * keep_first positions.  k_stride / v_stride: elements between cache rows (>= kv_heads dk / kv_heads dv; the value rows may
  * be a column range of the key rows); out_stride: elements between output rows (>= heads dv).  cap > 0: scaled scores become
  * cap tanh(score / cap); dist_bias (fp32 [heads][dist_n], or NULL): then dist_bias[h][min(tok_pos - key position, dist_n - 1)] is
- * added. */
+ * added.  head_gate (rows [n] of stride gate_ld, storage dtype, or NULL): head h's result times sigmoid(head_gate[t][h]). */
 int ll_ragged_attention(const void* q, const void* k_cache, const void* v_cache, const int32_t* token_table,
                         int64_t tt_stride, const int32_t* seq_req, const int32_t* tok_seq, const int32_t* tok_pos,
                         const void* sink, float scale, void* out, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk,
                         int64_t dv, int64_t k_stride, int64_t v_stride, int64_t window, int64_t keep_first,
-                        int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, int dtype, void* stream);
+                        int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, const void* head_gate,
+                        int64_t gate_ld, int dtype, void* stream);
 /* Rows [q (heads dk) | k (kv_heads dk) | v (kv_heads dv)] of stride ld, channel by channel in fp32: + bias [channels] (or NULL);
  * y_t = sum_j conv_w[c][j] u_(t - taps + 1 + j) over the sequence's positions (zeros in front of position 0; taps == 0: none),
  * the raw rows of a sequence's last taps - 1 positions carried in conv_state [2][state_half] (half seq_parity read, the other
@@ -622,7 +623,7 @@ int ll_ragged_attention(const void* q, const void* k_cache, const void* v_cache,
  * rotated by pos * freq[i] with cos / sin times amp (rot_table, when given, holds exactly these per token: ll_rotation_table;
  * the 16-byte form needs it); q / k heads divided by sqrt(mean + eps) when unit_norm; v = (1 - lam) v +
  * lam v_src[select[t]] when v_src (rows of stride v_src_stride; lam = *v_lam) is given.  q -> q_out [n, heads, dk]; k, v ->
- * cache rows select[t]. */
+ * cache rows select[t].  kv_heads == 0: rows hold queries only (no caches are written). */
 /* out [n][2 * pairs4] (fp32), pairs4 = pairs rounded up to a multiple of 4: entry pair i of token t at [t][2 i] =
  * (cos(tok_pos[t] * freq[i]) * amp, sin(tok_pos[t] * freq[i]) * amp); the padding is zero. */
 int ll_rotation_table(const int32_t* tok_pos, const float* freq, int64_t pairs, float amp, float* out, int64_t n, void* stream);
@@ -646,7 +647,7 @@ int ll_ragged_attention_mfma(const void* q, const void* k_cache, const void* v_c
                              int64_t batch, int64_t longest_run, int64_t longest_context, int decode, float* partials,
                              int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv, int64_t k_stride, int64_t v_stride,
                              int64_t window, int64_t keep_first, int64_t out_stride, float cap, const float* dist_bias,
-                             int64_t dist_n, int dtype, void* stream);
+                             int64_t dist_n, const void* head_gate, int64_t gate_ld, int dtype, void* stream);
 
 /* ---- sublayers between two grouped norms with a gated residual branch (csrc/group_norm.hip) --------------------------------
  * ll_gated_group_norm: with y: s = (sum of `parts` rows y[t][p][:] + shared_scale[t] * shared[t][:]) * sigmoid(gate[t][:] +
@@ -710,7 +711,8 @@ int ll_rotate_pairs(const void* q, int64_t q_tok_stride, int64_t q_head_stride, 
  * softmax over all logits; ranked by score + correction[e] (storage dtype, or NULL); weights = the chosen scores themselves;
  * the last `identity` experts return the token's own row: their slots keep ids >= experts - identity (never placed by
  * ll_moe_sort over the experts that have weights) and extra_scale[t] receives the sum of their scores.  scoring 3: as 0, but the
- * weights are the chosen sigmoid scores themselves.
+ * weights are the chosen sigmoid scores themselves.  scoring 4: scores = softmax over all logits, a group's score is its largest,
+ * weights as in 0.
  * ll_moe_sort: slots sorted by expert in blocks of `block` = ll_moe_rows_block(...) rows, 32 or 128 (counts: int32 scratch
  * [experts]; sorted [num_slots + experts (block - 1)], block_expert [ceil(that / block)], num_post [1]).
  * ll_moe_rows_gemm: glu != 0: w [experts][2 N][K] (gate rows, then up rows), out[slot] = silu(a Wg^T) * (a Wu^T) with
@@ -780,6 +782,19 @@ int ll_delta_scan(const void* q, int64_t q_ld, const void* k, int64_t k_ld, cons
                   const void* dt_bias, const void* a_log, const void* beta, int64_t beta_ld, float* o, int64_t batch,
                   const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, float* state,
                   float* scratch, int64_t n, int dtype, void* stream);
+
+/* ---- retention (csrc/retention.hip) ---------------------------------------------------------------------------------------------
+ * Per head, fp32 state [slots, heads, dk, dv]: q, k rotated (entry i < half with entry i + half, by (cos, sin) = rot[t][2 i], [2 i + 1]),
+ * k times k_scale; S <- decay[h] S + k v^T, o = S^T q.  A run that starts at position 0 starts from zeros.  o given (fp32 [n, heads
+ * dv]): runs of any length in chunks on the fp32 matrix cores, o is the read-out.  o NULL: every sequence brings one token (n ==
+ * batch); out rows (stride out_ld) = heads divided by sqrt(mean(o^2) + eps), times silu(gate) (rows of stride gate_ld, or NULL).
+ * dk <= 256. */
+int ll_retention_supported(int64_t dk, int64_t dv);
+int ll_retention(const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, int64_t heads,
+                 int64_t dk, int64_t dv, const float* rot, int64_t rot_ld, int64_t half, float k_scale, const float* decay,
+                 const int32_t* seq_start, const int32_t* seq_first_pos, const int32_t* seq_slot, float* state, float* o,
+                 const void* gate, int64_t gate_ld, float eps, void* out, int64_t out_ld, int64_t n, int64_t batch,
+                 int dtype, void* stream);
 
 /* ---- several mixed residual streams (csrc/stream_norm.hip) --------------------------------------------------------------------
  * With y: d = (sum of `parts` rows y[t][p][:] + shared_scale[t] * shared[t][:]) * scale (shared, scale may be NULL) and

@@ -118,12 +118,12 @@ SIGNATURES = {
     "ll_gated_linear_scan_supported": [L, L],
     "ll_gated_linear_scan": [P, P, P, L, P, P, P, F, P, L, L, L, L, P, P, P, P, L, L, P, I, P],
     "ll_qk_norm_cache": [P, L, P, P, F, F, L, P, P, P, P, P, L, L, L, L, L, I, P],
-    "ll_ragged_attention": [P, P, P, P, L, P, P, P, P, F, P, L, L, L, L, L, L, L, L, L, L, F, P, L, I, P],
+    "ll_ragged_attention": [P, P, P, P, L, P, P, P, P, F, P, L, L, L, L, L, L, L, L, L, L, F, P, L, P, L, I, P],
     "ll_rotation_table": [P, P, L, F, P, L, P],
     "ll_conv_rope_cache": [P, L, P, P, L, P, L, P, L, F, P, I, F, P, L, P, P, P, P, P, P, P, P, P, P, P, L, L, L, L, L, I, P],
     "ll_ragged_attention_mfma_supported": [L, L, I],
     "ll_ragged_attention_partition": [],
-    "ll_ragged_attention_mfma": [P, P, P, P, L, P, P, P, P, F, P, L, L, L, L, I, P, L, L, L, L, L, L, L, L, L, F, P, L, I, P],
+    "ll_ragged_attention_mfma": [P, P, P, P, L, P, P, P, P, F, P, L, L, L, L, I, P, L, L, L, L, L, L, L, L, L, F, P, L, P, L, I, P],
     "ll_gated_group_norm": [P, P, P, P, L, P, P, P, L, P, P, P, L, L, L, F, P, I, P],
     "ll_glu_act": [P, L, P, L, P, L, L, L, I, F, F, I, P],
     "ll_softcap": [P, L, F, I, P],
@@ -137,6 +137,8 @@ SIGNATURES = {
     "ll_moe_rows_gemm": [P, L, L, P, L, L, L, I, P, P, L, P, P, P, L, L, L, F, I, P],
     "ll_linear_scan_supported": [L, L],
     "ll_linear_scan": [P, L, P, L, P, L, L, L, L, L, I, I, F, P, P, L, P, F, P, L, P, P, P, P, L, P, P, P, P, P, L, L, I, P],
+    "ll_retention_supported": [L, L],
+    "ll_retention": [P, L, P, L, P, L, L, L, L, P, L, L, F, P, P, P, P, P, P, P, L, F, P, L, L, L, I, P],
     "ll_gated_out_norm": [P, L, P, P, L, I, I, P, L, F, F, L, L, L, I, P],
     "ll_conv_act": [P, L, P, L, P, P, L, L, P, L, P, P, P, P, P, P, L, I, I, P],
     "ll_rownorm_rope_cache": [P, L, P, P, F, P, L, F, P, P, P, P, P, L, L, L, L, L, I, P],

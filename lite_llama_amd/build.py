@@ -31,12 +31,13 @@ _NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 FILE_FLAGS = {"gemm_short.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=16"],
               "seq_mix.hip": _NO_PACKED_FP32, "ragged_attn.hip": _NO_PACKED_FP32, "ragged_attn_mfma.hip": _NO_PACKED_FP32,
               "group_norm.hip": _NO_PACKED_FP32, "latent_attn.hip": _NO_PACKED_FP32, "moe_sparse.hip": _NO_PACKED_FP32,
-              "linear_mix.hip": _NO_PACKED_FP32, "delta_scan.hip": _NO_PACKED_FP32, "stream_norm.hip": _NO_PACKED_FP32}
+              "linear_mix.hip": _NO_PACKED_FP32, "delta_scan.hip": _NO_PACKED_FP32, "stream_norm.hip": _NO_PACKED_FP32,
+              "retention.hip": _NO_PACKED_FP32}
 
 
 # part libraries: the sources ONE model family needs (a fresh checkout serving only that family builds nothing else)
 PARTS = {"ragged": ["seq_mix.hip", "ragged_attn.hip", "ragged_attn_mfma.hip", "group_norm.hip", "latent_attn.hip", "moe_sparse.hip",
-                    "linear_mix.hip", "delta_scan.hip", "stream_norm.hip", "kv_paged.hip", "kv_ops.hip", "sampler.hip"]}
+                    "linear_mix.hip", "delta_scan.hip", "stream_norm.hip", "retention.hip", "kv_paged.hip", "kv_ops.hip", "sampler.hip"]}
 
 
 def flags_for(src: str) -> list[str]:

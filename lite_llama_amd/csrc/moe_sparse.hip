@@ -132,7 +132,8 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const void* __restri
 // experts are ranked by score + correction[e], the weights are the chosen scores themselves (not renormalised); the last
 // `identity` experts have no weights of their own -- a slot that chose one keeps its id (>= experts - identity, which the sort
 // by expert never places) and its score is added to extra_scale[t], the factor of the token's own input row; 3: sigmoid scores
-// as in 0, but the weights are the chosen scores themselves (not renormalised)
+// as in 0, but the weights are the chosen scores themselves (not renormalised); 4: scores = softmax over ALL logits, a group's score is
+// its largest, weights = chosen / sum
 template <int SCORING, int DT = LL_F32>
 __global__ __launch_bounds__(64) void group_select_kernel(const float* __restrict__ logits, int rows, int experts, int top,
                                                           int group_count, int group_keep, float route_scale,
@@ -184,10 +185,19 @@ __global__ __launch_bounds__(64) void group_select_kernel(const float* __restric
   }
   for (int e = lane; e < rows; e += 64) {
     const float z = logits[t * rows + e];
-    if (e < experts) score[e] = SCORING == 1 ? z : sigmoid_exact(z);
+    if (e < experts) score[e] = (SCORING == 1 || SCORING == 4) ? z : sigmoid_exact(z);
     else extra_scale[t] = sigmoid_exact(z);
   }
   __syncthreads();
+  if constexpr (SCORING == 4) {   // the logits become softmax scores: every lane adds all exponentials in index order
+    float top_z = -INFINITY;
+    for (int e = 0; e < experts; ++e) top_z = fmaxf(top_z, score[e]);
+    float total = 0.f;
+    for (int e = 0; e < experts; ++e) total += expf(score[e] - top_z);
+    __syncthreads();
+    for (int e = lane; e < experts; e += 64) score[e] = expf(score[e] - top_z) / total;
+    __syncthreads();
+  }
   const int per = experts / group_count;
   for (int g = lane; g < group_count; g += 64) {
     float b1 = -INFINITY, b2 = -INFINITY;   // the two largest of the group
@@ -196,7 +206,7 @@ __global__ __launch_bounds__(64) void group_select_kernel(const float* __restric
       if (s > b1) { b2 = b1; b1 = s; }
       else if (s > b2) b2 = s;
     }
-    gscore[g] = per > 1 ? b1 + b2 : b1;
+    gscore[g] = SCORING != 4 && per > 1 ? b1 + b2 : b1;
   }
   __syncthreads();
   for (int g = lane; g < group_count; g += 64) {
@@ -560,7 +570,7 @@ extern "C" int ll_group_router(const void* h, int64_t h_ld, const void* w_router
   if (scoring != 2 && (correction || identity)) return LL_ERR_SHAPE;
   if (n < 0 || width < 1 || h_ld < width || experts < 1 || experts > 4096 || top < 1 || top > experts || top > 64 || group_count < 1 ||
       experts % group_count || group_keep < 1 || group_keep > group_count || group_keep * (experts / group_count) < top ||
-      scoring < 0 || scoring > 3 || (scoring == 1 && group_count != 1))
+      scoring < 0 || scoring > 4 || (scoring == 1 && group_count != 1))
     return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
   if (!h || !w_router || !ids || !weights || !logits || (w_extra && !extra_scale)) return LL_ERR_ARG;
@@ -596,6 +606,9 @@ extern "C" int ll_group_router(const void* h, int64_t h_ld, const void* w_router
 #undef CALL
   } else if (scoring == 1)
     group_select_kernel<1><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,
+                                                               route_scale, ids, weights, extra_scale);
+  else if (scoring == 4)
+    group_select_kernel<4><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,
                                                                route_scale, ids, weights, extra_scale);
   else if (scoring == 3)
     group_select_kernel<3><<<dim3((unsigned)n), 64, lds, st>>>(logits, rows, (int)experts, (int)top, (int)group_count, (int)group_keep,

@@ -13,7 +13,7 @@
 //   ll_ragged_attention  every token of the step against keys 0 .. its own position of its sequence, read through the
 //                        per-token row table; scores, softmax and the running output in fp32; optionally only the last
 //                        `window` keys plus the sequence's first `keep_first`; optionally scores capped to cap tanh(s / cap)
-//                        and a bias per head and distance added
+//                        and a bias per head and distance added, a head's result times the sigmoid of its gate logit
 //
 // The sink is a virtual key with score sink_h (not scaled) and a zero value: the running softmax simply STARTS at
 // (max = sink, sum = 1, output = 0).  A token's result depends only on its own position and on the cache rows of its
@@ -477,6 +477,14 @@ __device__ __forceinline__ float dot_row(const float* __restrict__ a, const void
   return d;
 }
 
+// sigmoid of a head's gate logit: libm's exp for fp32 storage, the hardware exp2 / reciprocal (1 ulp each) for 16-bit storage
+template <int DT>
+__device__ __forceinline__ float head_gate_factor(const void* gate, int64_t at) {
+  const float z = ldv<DT>(gate, at);
+  if constexpr (DT == LL_F32) return 1.0f / (1.0f + expf(-z));
+  else return ll_sigmoidf(z);
+}
+
 // One wave per (token, query head).  Keys in tiles of 64: lane j scores key base + j (a contiguous dk-row of the cache),
 // the tile's weights go through LDS, then lane c accumulates channel c (and c + 64, ...) of the output over the tile.
 template <int DT, int VPL>
@@ -485,7 +493,8 @@ __global__ __launch_bounds__(256) void ragged_attention_kernel(
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos, const void* __restrict__ sink, float scale,
     void* __restrict__ out, int64_t n, int heads, int kv_heads, int dk, int dv, int64_t k_stride, int64_t v_stride, int window,
-    int keep_first, int64_t out_stride, float cap, const float* __restrict__ dist_bias, int dist_n) {
+    int keep_first, int64_t out_stride, float cap, const float* __restrict__ dist_bias, int dist_n,
+    const void* __restrict__ head_gate, int64_t gate_ld) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   float* sq = lds + wave * (dk + 128);  // [dk] query
@@ -546,7 +555,8 @@ __global__ __launch_bounds__(256) void ragged_attention_kernel(
     }
     __builtin_amdgcn_wave_barrier();
   }
-  const float inv = 1.0f / l;
+  float inv = 1.0f / l;
+  if (head_gate) inv *= head_gate_factor<DT>(head_gate, t * gate_ld + h);
 #pragma unroll
   for (int i = 0; i < VPL; ++i) {
     const int c = lane + 64 * i;
@@ -629,12 +639,13 @@ extern "C" int ll_conv_rope_cache(const void* qkv, int64_t ld, const void* bias,
                                   void* k_cache, void* v_cache, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv,
                                   int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
-  if (n < 0 || heads < 1 || kv_heads < 1 || heads % kv_heads || dk < 1 || dk > 1024 || dv < 1 || dv > 1024 || taps < 0 || taps > 64 ||
+  // (no key/value heads: rows hold queries only, the keys and values they meet are another layer's)
+  if (n < 0 || heads < 1 || kv_heads < 0 || (kv_heads && heads % kv_heads) || dk < 1 || dk > 1024 || dv < 1 || dv > 1024 || taps < 0 || taps > 64 ||
       pairs < 0 || 2 * pairs > dk || ld < (heads + kv_heads) * dk + kv_heads * dv || (v_src && v_src_stride < kv_heads * dv))
     return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
-  if (!qkv || !tok_seq || !tok_pos || !select || !seq_start || !seq_first_pos || !seq_slot || !seq_parity || !q_out || !k_cache ||
-      !v_cache || (taps > 0 && !conv_w) || (taps > 1 && !conv_state) || (pairs > 0 && !freq && !rot_table) || (v_src && !v_lam))
+  if (!qkv || !tok_seq || !tok_pos || !select || !seq_start || !seq_first_pos || !seq_slot || !seq_parity || !q_out ||
+      (kv_heads && (!k_cache || !v_cache)) || (taps > 0 && !conv_w) || (taps > 1 && !conv_state) || (pairs > 0 && !freq && !rot_table) || (v_src && !v_lam))
     return LL_ERR_ARG;
   const int64_t waves = n * (heads + 2 * kv_heads);
   const dim3 grid((unsigned)((waves + 3) / 4));
@@ -690,11 +701,12 @@ extern "C" int ll_ragged_attention(const void* q, const void* k_cache, const voi
                                    int64_t tt_stride, const int32_t* seq_req, const int32_t* tok_seq, const int32_t* tok_pos,
                                    const void* sink, float scale, void* out, int64_t n, int64_t heads, int64_t kv_heads, int64_t dk,
                                    int64_t dv, int64_t k_stride, int64_t v_stride, int64_t window, int64_t keep_first,
-                                   int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, int dtype, void* stream) {
+                                   int64_t out_stride, float cap, const float* dist_bias, int64_t dist_n, const void* head_gate, int64_t gate_ld,
+                                   int dtype, void* stream) {
   if (dtype != LL_F16 && dtype != LL_BF16 && dtype != LL_F32) return LL_ERR_DTYPE;
   if (n < 0 || heads < 1 || kv_heads < 1 || heads % kv_heads || dk < 1 || dk > 1024 || dv < 1 || dv > 1024 || window < 0 ||
       window > 0x7fffffff || keep_first < 0 || keep_first > 0x7fffffff || k_stride < kv_heads * dk || v_stride < kv_heads * dv ||
-      out_stride < heads * dv || !(cap >= 0.f) || (dist_bias && (dist_n < 1 || dist_n > 0x7fffffff)))
+      out_stride < heads * dv || !(cap >= 0.f) || (dist_bias && (dist_n < 1 || dist_n > 0x7fffffff)) || (head_gate && gate_ld < heads))
     return LL_ERR_SHAPE;
   if (n == 0) return LL_OK;
   if (!q || !k_cache || !v_cache || !token_table || !seq_req || !tok_seq || !tok_pos || !out) return LL_ERR_ARG;
@@ -706,7 +718,7 @@ extern "C" int ll_ragged_attention(const void* q, const void* k_cache, const voi
 #define CALL_V(DT, V)                                                                                                        \
   ragged_attention_kernel<DT, V><<<grid, 256, lds, st>>>(q, k_cache, v_cache, token_table, tt_stride, seq_req, tok_seq, tok_pos, \
                                                          sink, scale, out, n, (int)heads, (int)kv_heads, (int)dk, (int)dv, k_stride, \
-                                                         v_stride, (int)window, (int)keep_first, out_stride, cap, dist_bias, (int)dist_n)
+                                                         v_stride, (int)window, (int)keep_first, out_stride, cap, dist_bias, (int)dist_n, head_gate, gate_ld)
 #define CALL(DT)                     \
   if (vpl == 1) CALL_V(DT, 1);       \
   else if (vpl == 2) CALL_V(DT, 2);  \

@@ -14,6 +14,7 @@
 // Widths that are not multiples of 32 (keys) / 16 (values) are zero-padded; both must be multiples of 8.
 // BIASED forms: scores capped to cap tanh(s / cap), then a bias per head and distance (dist_bias [heads][dist_n], fp32; distances
 // beyond the table read its last entry) is added; the softmax runs in base 2, so both enter times log2(e).
+// A head's result may be multiplied by the sigmoid of its gate logit where it is stored.
 #include "common.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -51,6 +52,16 @@ struct ScoreShape {
   int dist_n;
 };
 
+// logits [n][ld] of one gate per token and head (NULL: none): a head's result is multiplied by the sigmoid of its logit
+struct HeadGate {
+  const uint16_t* z;
+  int64_t ld;
+};
+template <int DT>
+__device__ __forceinline__ float gate_factor(const HeadGate& g, int64_t token, int head) {
+  return g.z ? ll_sigmoidf(to_f32<DT>(g.z[token * g.ld + head])) : 1.0f;
+}
+
 // scaled dot product -> capped, biased score times log2(e); tanh(x) = 1 - 2 / (1 + e^(2x)) through the hardware exp2 / reciprocal
 __device__ __forceinline__ float shaped_score(float dot, const ScoreShape& sh, float bias) {
   float s = dot * sh.scale;
@@ -68,7 +79,8 @@ __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ seq_start, const int32_t* __restrict__ seq_first_pos, const uint16_t* __restrict__ sink,
     float scale_log2, uint16_t* __restrict__ out, float* __restrict__ partials, int max_parts, int heads, int kv_heads, int dk,
-    int dv, int64_t k_stride, int64_t v_stride, int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape) {
+    int dv, int64_t k_stride, int64_t v_stride, int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape,
+    HeadGate gate) {
   static_assert(NTM / 2 == NSM, "value fragments of shared rows are the key fragments");
   constexpr int QB = 1;
   constexpr bool DECODE = true;
@@ -300,7 +312,7 @@ __global__ __launch_bounds__(64) void ragged_attention_mfma_decode_kernel(
   for (int qb = 0; qb < QB; ++qb) {
     if (!valid[qb]) continue;
     if (!DECODE || max_parts == 1) {
-      const float inv = 1.0f / d_i[qb];
+      const float inv = gate_factor<DT>(gate, token[qb], head[qb]) / d_i[qb];
       uint16_t* o = out + (int64_t)token[qb] * out_stride + (int64_t)head[qb] * dv;
 #pragma unroll
       for (int dt = 0; dt < NTM; ++dt) {
@@ -340,7 +352,7 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
     const int32_t* __restrict__ token_table, int64_t tt_stride, const int32_t* __restrict__ seq_req,
     const int32_t* __restrict__ seq_start, const int32_t* __restrict__ seq_first_pos, const uint16_t* __restrict__ sink,
     float scale_log2, uint16_t* __restrict__ out, int heads, int kv_heads, int dk, int dv, int64_t k_stride, int64_t v_stride,
-    int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape) {
+    int window, int shared_kv, int keep_first, int64_t out_stride, ScoreShape shape, HeadGate gate) {
   constexpr int KSTR = NSM * 32 + 8, VSTR = NTM * 16 + 8;
   constexpr int KPASS = (32 * NSM * 4 + 255) / 256, VPASS = (32 * NTM * 2 + 255) / 256;  // 16-byte pieces per thread
   __shared__ __attribute__((aligned(16))) uint16_t lds_k[32 * KSTR];
@@ -534,7 +546,7 @@ __global__ __launch_bounds__(256) void ragged_attention_mfma_prefill4_kernel(
 #undef LL_FETCH
 #undef LL_STAGE
   if (!valid) return;
-  const float inv = 1.0f / d_i;
+  const float inv = gate_factor<DT>(gate, token, head) / d_i;
   uint16_t* o = out + (int64_t)token * out_stride + (int64_t)head * dv;
 #pragma unroll
   for (int dt = 0; dt < NTM; ++dt) {
@@ -551,7 +563,7 @@ template <int DT>
 __global__ __launch_bounds__(256) void ragged_attention_merge_kernel(const float* __restrict__ partials, int max_parts,
                                                                      const int32_t* __restrict__ seq_first_pos,
                                                                      uint16_t* __restrict__ out, int64_t n, int heads, int dv,
-                                                                     int window, int keep_first, int64_t out_stride) {
+                                                                     int window, int keep_first, int64_t out_stride, HeadGate gate) {
   const int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (w >= n * heads) return;
   const int lane = threadIdx.x & 63;
@@ -570,11 +582,12 @@ __global__ __launch_bounds__(256) void ragged_attention_merge_kernel(const float
   for (int p = 0; p < parts; ++p)
     if (p >= p_lo || p < p_kept) d += src[p * (2 + dv) + 1] * exp2f(src[p * (2 + dv)] - m);
   const int h = (int)(w - token * heads);
+  const float factor = gate_factor<DT>(gate, token, h);
   for (int ch = lane; ch < dv; ch += 64) {
     float o = 0.f;
     for (int p = 0; p < parts; ++p)
       if (p >= p_lo || p < p_kept) o += src[p * (2 + dv) + 2 + ch] * exp2f(src[p * (2 + dv)] - m);
-    out[token * out_stride + (int64_t)h * dv + ch] = from_f32<DT>(o / d);
+    out[token * out_stride + (int64_t)h * dv + ch] = from_f32<DT>(o / d * factor);
   }
 }
 
@@ -595,11 +608,11 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
                                         int64_t batch, int64_t longest_run, int64_t longest_context, int decode, float* partials,
                                         int64_t heads, int64_t kv_heads, int64_t dk, int64_t dv, int64_t k_stride, int64_t v_stride,
                                         int64_t window, int64_t keep_first, int64_t out_stride, float cap, const float* dist_bias,
-                                        int64_t dist_n, int dtype, void* stream) {
+                                        int64_t dist_n, const void* head_gate, int64_t gate_ld, int dtype, void* stream) {
   if (!ll_ragged_attention_mfma_supported(dk, dv, dtype)) return dtype == LL_F32 ? LL_ERR_DTYPE : LL_ERR_SHAPE;
   if (k_stride < kv_heads * dk || v_stride < kv_heads * dv || k_stride % 8 || v_stride % 8 || window < 0 || window > 0x7fffffff ||
       keep_first < 0 || keep_first > 0x7fffffff || out_stride < heads * dv ||
-      !ll_aligned16(k_cache) || !ll_aligned16(v_cache) || !ll_aligned16(q))
+      (head_gate && gate_ld < heads) || !ll_aligned16(k_cache) || !ll_aligned16(v_cache) || !ll_aligned16(q))
     return LL_ERR_SHAPE;
   if (n < 0 || batch < 0 || heads < 1 || kv_heads < 1 || heads % kv_heads || heads > 65535 || batch > 65535 || longest_run < 1 ||
       longest_context < 1 || (decode && n != batch))
@@ -615,12 +628,13 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
   const float scale_log2 = scale * kLog2e;
   if (!(cap >= 0.f) || (dist_bias && (dist_n < 1 || dist_n > 0x7fffffff))) return LL_ERR_SHAPE;
   const bool biased = cap > 0.f || dist_bias;
+  const HeadGate gate = {(const uint16_t*)head_gate, gate_ld};
   const ScoreShape shape = {scale, cap, dist_bias, dist_bias ? (int)dist_n : 1};
 #define CALL_DB(DT, NS, NT, B)                                                                                                   \
   ragged_attention_mfma_decode_kernel<DT, NS, NT, B><<<grid, 64, 0, st>>>(                                                      \
       (const uint16_t*)q, (const uint16_t*)k_cache, (const uint16_t*)v_cache, token_table, tt_stride, seq_req, seq_start,    \
       seq_first_pos, (const uint16_t*)sink, scale_log2, (uint16_t*)out, partials, max_parts, (int)heads, (int)kv_heads, (int)dk, \
-      (int)dv, k_stride, v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape)
+      (int)dv, k_stride, v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape, gate)
 #define CALL_D(DT, NS, NT)                         \
   if (biased) { CALL_DB(DT, NS, NT, true); }       \
   else { CALL_DB(DT, NS, NT, false); }
@@ -634,7 +648,7 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
   ragged_attention_mfma_prefill4_kernel<DT, NS, NT, B><<<grid4, 256, 0, st>>>(                                                 \
       (const uint16_t*)q, (const uint16_t*)k_cache, (const uint16_t*)v_cache, token_table, tt_stride, seq_req, seq_start,   \
       seq_first_pos, (const uint16_t*)sink, scale_log2, (uint16_t*)out, (int)heads, (int)kv_heads, (int)dk, (int)dv, k_stride,   \
-      v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape)
+      v_stride, (int)window, shared_kv, (int)keep_first, out_stride, shape, gate)
 #define CALL_4(DT, NS, NT)                         \
   if (biased) { CALL_4B(DT, NS, NT, true); }       \
   else { CALL_4B(DT, NS, NT, false); }
@@ -656,10 +670,10 @@ extern "C" int ll_ragged_attention_mfma(const void* q, const void* k_cache, cons
     const int64_t waves = n * heads;
     if (dtype == LL_F16)
       ragged_attention_merge_kernel<LL_F16><<<dim3((unsigned)((waves + 3) / 4)), 256, 0, st>>>(partials, max_parts, seq_first_pos,
-                                                                                            (uint16_t*)out, n, (int)heads, (int)dv, (int)window, (int)keep_first, out_stride);
+                                                                                            (uint16_t*)out, n, (int)heads, (int)dv, (int)window, (int)keep_first, out_stride, gate);
     else
       ragged_attention_merge_kernel<LL_BF16><<<dim3((unsigned)((waves + 3) / 4)), 256, 0, st>>>(partials, max_parts, seq_first_pos,
-                                                                                             (uint16_t*)out, n, (int)heads, (int)dv, (int)window, (int)keep_first, out_stride);
+                                                                                             (uint16_t*)out, n, (int)heads, (int)dv, (int)window, (int)keep_first, out_stride, gate);
   }
   return LL_LAUNCH_CHECK();
 }

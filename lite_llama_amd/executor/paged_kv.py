@@ -100,7 +100,7 @@ class PagedStateCache(PagedKVPool):
     own a token-shift row pair ``[2, slots, width]`` (double-buffered by the sequence's parity).  A run with a short
     convolution in front of it (attention or recurrence) carries the projected rows of a sequence's last positions, ``[2, slots, taps - 1, channels]``,
     double-buffered the same way; a run whose values are blended with those of an earlier run names that run in
-    ``value_source``; a model whose input depends on the previous token keeps it per sequence in ``prev_token [2, slots]``.  One block allocator, one
+    ``value_source``; a run that reads an earlier run's keys and values lists that run's buffers as its own; a model whose input depends on the previous token keeps it per sequence in ``prev_token [2, slots]``.  One block allocator, one
     block table and one per-token row table serve all attention runs; a sequence's slot is its row of those tables, so blocks
     and slots are handed out and given back together.  Fixed-size state is never cleared: the kernels start a sequence whose
     run begins at position 0 from zeros, whatever an earlier owner of the slot left."""
@@ -108,7 +108,8 @@ class PagedStateCache(PagedKVPool):
     def __init__(self, runs, num_blocks: int, block_size: int, device, max_requests: int, max_seq_len: int, dtype,
                  previous_token: bool = False):
         """``runs``: one mapping per layer run: ``{"kind": "attention", "kv_heads", "dk", "dv"}``, ``{"kind": "latent", "rank",
-        "rot"}`` or ``{"kind": "recurrent", "heads", "dk", "dv"}``, each with an optional ``"shift_width"``; attention and recurrent runs
+        "rot"}`` ``{"kind": "recurrent", "heads", "dk", "dv"}`` or ``{"kind": "shared", "source": run}`` (the keys and values of an earlier attention
+        run, nothing of its own), each with an optional ``"shift_width"``; attention and recurrent runs
         may add ``"conv_taps"`` / ``"conv_channels"`` (rows carried for a convolution of that many taps), attention runs ``"value_mix": True``
         (the first such run is the value source of the later ones) and ``"state": (heads, dk, dv)`` (a recurrence that runs
         beside the attention keeps its fp32 state in the same run).  ``previous_token``: keep each sequence's last token."""
@@ -141,6 +142,13 @@ class PagedStateCache(PagedKVPool):
                 # latent columns of the same rows (a row-strided view, nothing is stored twice)
                 rows = torch.zeros(self.max_tokens, 1, r["rank"] + r["rot"], dtype=dtype, device=dev)
                 buffers.append((rows, rows[:, :, :r["rank"]]))
+                self.recurrent.append(None)
+            elif r["kind"] == "shared":
+                # reads what an earlier attention run has cached; keeps nothing of its own
+                source = int(r["source"])
+                if not (0 <= source < index and self.runs[source]["kind"] == "attention"):
+                    raise ValueError(f"layer run {index} shares the cache of run {source}, which is not an earlier attention run")
+                buffers.append(buffers[source])
                 self.recurrent.append(None)
             elif r["kind"] == "recurrent":
                 buffers.append(None)

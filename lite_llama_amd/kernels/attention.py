@@ -333,15 +333,15 @@ def conv_rope_cache(qkv, heads: int, kv_heads: int, dk: int, dv: int, step, k_ca
     sequence's parity is read, the other written); entry pairs ``(2i, 2i + 1)``, ``i < pairs``, of every q / k head rotated by
     ``position * freq[i]`` with cos / sin times ``amp``; q / k heads divided by ``sqrt(mean + eps)`` when ``unit_norm``; values
     become ``(1 - b) v + b v_source[select]`` when ``v_source [rows, kv_heads, dv]`` (another layer's value cache) and the
-    one-element tensor ``v_blend`` are given.  ``rot_table``: :func:`rotation_table` of this step for these frequencies (made
+    one-element tensor ``v_blend`` are given.  ``kv_heads = 0`` (no caches): rows hold queries only.  ``rot_table``: :func:`rotation_table` of this step for these frequencies (made
     here when absent; layers that rotate alike share one)."""
     L.require_cuda(qkv, k_cache, v_cache, bias, conv_weight, conv_state, freq, v_source, v_blend)
     n, dt = qkv.shape[0], qkv.dtype
     channels = (heads + kv_heads) * dk + kv_heads * dv
     if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < channels or step.num_tokens != n:
         raise ValueError("conv_rope_cache: rows hold [q | k | v] of the step's tokens")
-    if k_cache.dtype != dt or v_cache.dtype != dt or tuple(k_cache.shape[1:]) != (kv_heads, dk) \
-            or tuple(v_cache.shape[1:]) != (kv_heads, dv) or not (k_cache.is_contiguous() and v_cache.is_contiguous()):
+    if kv_heads and (k_cache.dtype != dt or v_cache.dtype != dt or tuple(k_cache.shape[1:]) != (kv_heads, dk)
+                     or tuple(v_cache.shape[1:]) != (kv_heads, dv) or not (k_cache.is_contiguous() and v_cache.is_contiguous())):
         raise ValueError("conv_rope_cache: caches are contiguous [rows, kv_heads, dk] / [rows, kv_heads, dv] in the rows' dtype")
     if bias is not None and (bias.dtype != dt or bias.numel() != channels or not bias.is_contiguous()):
         raise ValueError("conv_rope_cache: one bias per channel, in the rows' dtype")
@@ -372,8 +372,8 @@ def conv_rope_cache(qkv, heads: int, kv_heads: int, dk: int, dv: int, step, k_ca
         L.ptr(v_source),
         v_source.stride(0) if v_source is not None else 0, L.ptr(v_blend) if v_source is not None else 0, step.tok_seq.data_ptr(),
         step.tok_pos.data_ptr(), step.select.data_ptr(), step.seq_start.data_ptr(), step.seq_first_pos.data_ptr(),
-        step.seq_slot.data_ptr(), step.seq_parity.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), n, heads,
-        kv_heads, dk, dv, L.dtype_code(dt), L.stream_ptr()), "conv_rope_cache")
+        step.seq_slot.data_ptr(), step.seq_parity.data_ptr(), q.data_ptr(), L.ptr(k_cache) if kv_heads else 0,
+        L.ptr(v_cache) if kv_heads else 0, n, heads, kv_heads, dk, dv, L.dtype_code(dt), L.stream_ptr()), "conv_rope_cache")
     return q
 
 
@@ -409,14 +409,15 @@ def rownorm_rope_cache(qkv, heads: int, kv_heads: int, dk: int, dv: int, step, k
 
 @torch.no_grad()
 def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=None, window: int = 0, keep_first: int = 0,
-                     out=None, cap: float = 0.0, dist_bias=None):
+                     out=None, cap: float = 0.0, dist_bias=None, head_gate=None):
     """Causal softmax attention of every token of a ragged step against positions ``0 .. its own`` of its sequence, keys and
     values read through ``token_table[request][position]``; ``sink [heads]`` adds ``exp(sink_h)`` to each head's denominator;
     ``window > 0`` keeps the last ``window`` positions (the token's own included) and, besides them, the sequence's first
     ``keep_first`` positions.  ``k_cache [rows, kv_heads, dk]`` /
     ``v_cache [rows, kv_heads, dv]`` may be row-strided views (the values of a latent cache are a column range of its key
     rows).  ``cap > 0``: scaled scores become ``cap tanh(score / cap)``; ``dist_bias`` (fp32 ``[heads, m]``): then the entry of the
-    distance between token and key is added per head (distances from ``m - 1`` on read the last entry).  Scores, weights and the
+    distance between token and key is added per head (distances from ``m - 1`` on read the last entry).  ``head_gate [n, heads]`` (a row-strided
+    view): head h's result is multiplied by ``sigmoid(head_gate[t, h])``.  Scores, weights and the
     output sum are fp32.  Returns ``[n, heads * dv]`` (``out``: a view of that shape with a
     unit inner stride, e.g. a column range of the next projection's input)."""
     L.require_cuda(q, k_cache, v_cache, token_table)
@@ -435,7 +436,11 @@ def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=
     if dist_bias is not None and (dist_bias.dtype != torch.float32 or dist_bias.dim() != 2 or dist_bias.shape[0] != heads
                                   or dist_bias.shape[1] < 1 or not dist_bias.is_contiguous() or not dist_bias.is_cuda):
         raise ValueError("ragged_attention: the distance bias is fp32 [heads, distances]")
+    if head_gate is not None and (head_gate.dtype != dt or tuple(head_gate.shape) != (n, heads) or head_gate.stride(1) != 1
+                                  or not head_gate.is_cuda):
+        raise ValueError("ragged_attention: gate logits are [n, heads] in the queries' dtype with a unit inner stride")
     bias_n = dist_bias.shape[1] if dist_bias is not None else 0
+    gate_ld = max(head_gate.stride(0), heads) if head_gate is not None else 0
     if step.num_tokens != n:
         raise ValueError("ragged_attention: the step describes another number of tokens")
     ks, vs = k_cache.stride(0), v_cache.stride(0)
@@ -458,14 +463,14 @@ def ragged_attention(q, k_cache, v_cache, scale: float, step, token_table, sink=
             q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), token_table.data_ptr(), token_table.stride(0),
             step.seq_req.data_ptr(), step.seq_start.data_ptr(), step.seq_first_pos.data_ptr(), L.ptr(sink), float(scale),
             out.data_ptr(), n, step.num_seqs, step.longest_run, step.longest_context, 1 if decode else 0, L.ptr(scratch), heads,
-            kv_heads, dk, dv, ks, vs, int(window), int(keep_first), os_, float(cap), L.ptr(dist_bias), bias_n, L.dtype_code(dt),
-            L.stream_ptr()), "ragged_attention_mfma")
+            kv_heads, dk, dv, ks, vs, int(window), int(keep_first), os_, float(cap), L.ptr(dist_bias), bias_n, L.ptr(head_gate),
+            gate_ld, L.dtype_code(dt), L.stream_ptr()), "ragged_attention_mfma")
         return out
     L.check(L.lib().ll_ragged_attention(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), token_table.data_ptr(),
                                         token_table.stride(0), step.seq_req.data_ptr(), step.tok_seq.data_ptr(),
                                         step.tok_pos.data_ptr(), L.ptr(sink), float(scale), out.data_ptr(), n, heads, kv_heads, dk,
                                         dv, ks, vs, int(window), int(keep_first), os_, float(cap), L.ptr(dist_bias), bias_n,
-                                        L.dtype_code(dt), L.stream_ptr()),
+                                        L.ptr(head_gate), gate_ld, L.dtype_code(dt), L.stream_ptr()),
             "ragged_attention")
     return out
 

@@ -264,7 +264,8 @@ def group_router(h: torch.Tensor, router_weight: torch.Tensor, top: int, group_c
     renormalised.  The last ``identity`` router outputs stand for experts that return the token's own row: their slots keep
     ids ``>= experts - identity`` (which :func:`sparse_glu_experts` leaves as zero rows) and ``extra`` is the sum of their
     scores per token -- the factor of ``h`` itself in the sublayer's result.  ``scoring="sigmoid_plain"``: as ``"sigmoid"``, but the
-    weights are the chosen scores themselves (times ``route_scale``), not divided by their sum."""
+    weights are the chosen scores themselves (times ``route_scale``), not divided by their sum.  ``scoring="softmax_groups"``: scores are
+    the softmax over all router outputs, a group's score is its LARGEST, the weights are divided by their sum as in ``"sigmoid"``."""
     L.require_cuda(h, router_weight, extra_weight, correction)
     n, width = h.shape
     experts = router_weight.shape[0]
@@ -282,7 +283,7 @@ def group_router(h: torch.Tensor, router_weight: torch.Tensor, top: int, group_c
     logits = torch.empty(n, experts + (1 if extra_weight is not None else 0), dtype=torch.float32, device=h.device)
     L.check(L.lib().ll_group_router(h.data_ptr(), h.stride(0), router_weight.data_ptr(), L.ptr(extra_weight), n, width, experts,
                                     int(top), int(group_count), int(group_keep), float(route_scale),
-                                    {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2, "sigmoid_plain": 3}[scoring], ids.data_ptr(),
+                                    {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2, "sigmoid_plain": 3, "softmax_groups": 4}[scoring], ids.data_ptr(),
                                     weights.data_ptr(), L.ptr(extra), logits.data_ptr(), L.ptr(correction), int(identity),
                                     L.dtype_code(h.dtype), L.stream_ptr()),
             "group_router")

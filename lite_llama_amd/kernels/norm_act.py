@@ -573,13 +573,17 @@ def glu_act(gate: torch.Tensor, ff: int, kind: str, up: torch.Tensor | None = No
 
 
 @torch.no_grad()
-def relu_square(x: torch.Tensor, ff: int) -> torch.Tensor:
-    """``relu(x[:, :ff])^2`` of row-strided rows (fp32 arithmetic, one rounding to the storage dtype)."""
+def relu_square(x: torch.Tensor, ff: int, out: torch.Tensor | None = None) -> torch.Tensor:
+    """``relu(x[:, :ff])^2`` of row-strided rows (fp32 arithmetic, one rounding to the storage dtype).  ``out``: a ``[n, ff]`` view
+    with a unit inner stride (a column range of the next projection's input)."""
     L.require_cuda(x)
     if x.dim() != 2 or x.stride(1) != 1 or x.shape[1] < ff:
         raise ValueError("relu_square: rows are [n, >= ff] with a unit inner stride")
-    out = torch.empty(x.shape[0], ff, dtype=x.dtype, device=x.device)
-    L.check(L.lib().ll_glu_act(out.data_ptr(), ff, x.data_ptr(), max(x.stride(0), ff), 0, 0, x.shape[0], int(ff), 4, 0.0, 0.0,
+    if out is None:
+        out = torch.empty(x.shape[0], ff, dtype=x.dtype, device=x.device)
+    elif out.dtype != x.dtype or tuple(out.shape) != (x.shape[0], ff) or out.stride(1) != 1 or not out.is_cuda:
+        raise ValueError("relu_square: out is [n, ff] in the input's dtype with a unit inner stride")
+    L.check(L.lib().ll_glu_act(out.data_ptr(), max(out.stride(0), ff), x.data_ptr(), max(x.stride(0), ff), 0, 0, x.shape[0], int(ff), 4, 0.0, 0.0,
                                L.dtype_code(x.dtype), L.stream_ptr()), "relu_square")
     return out
 

@@ -238,6 +238,60 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: int, d
     return o
 
 
+# ------------------------------------------------------------------------------------- #
+# retention (csrc/retention.hip)
+# ------------------------------------------------------------------------------------- #
+def retention_supported(dk: int, dv: int) -> bool:
+    return bool(L.lib().ll_retention_supported(dk, dv))
+
+
+@torch.no_grad()
+def retention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: int, dk: int, dv: int, step, state: torch.Tensor, *,
+              decay: torch.Tensor, gate: torch.Tensor, eps: float, k_scale: float = 1.0, half: int = 0,
+              rot_table: torch.Tensor | None = None, out: torch.Tensor | None = None) -> torch.Tensor:
+    """Linear attention with a fixed decay per head over a ragged step: entry ``i < half`` of every q / k head is rotated with entry
+    ``i + half`` by the token's angles (``rot_table``: ``kernels.attention.rotation_table`` of this step), keys are multiplied by
+    ``k_scale``; per head ``S <- decay_h S + k_t v_t^T``, ``o_t = S^T q_t``; every head of ``o`` is divided by
+    ``sqrt(mean(o^2) + eps)`` and multiplied by ``silu(gate)``.  ``q`` / ``k`` / ``v`` / ``gate``: row-strided views ``[n, heads dk]`` /
+    ``[n, heads dv]`` (column ranges of a fused projection); ``decay`` fp32 ``[heads]``.  ``state [slots, heads, dk, dv]`` fp32: a sequence
+    whose run starts at position 0 starts from zeros, every run leaves its final state.  Rotation, state, read-out and norm are
+    fp32.  Returns ``[n, heads dv]`` in the storage dtype (``out``: a view of that shape with a unit inner stride).
+
+    Steps of one decoded token per sequence are one launch; runs of several tokens walk chunks on the fp32 matrix cores, then the
+    norm and the gate (:func:`gated_out_norm`)."""
+    L.require_cuda(q, k, v, state, decay, gate, rot_table, out)
+    n, st = q.shape[0], q.dtype
+    for t, cols, what in ((q, heads * dk, "query"), (k, heads * dk, "key"), (v, heads * dv, "value"), (gate, heads * dv, "gate")):
+        if t.dim() != 2 or t.stride(1) != 1 or t.shape[1] < cols or t.shape[0] != n or t.dtype != st:
+            raise ValueError(f"retention: {what} rows are [n, >= {cols}] of the queries' dtype with a unit inner stride")
+    if decay.dtype != torch.float32 or decay.numel() != heads or not decay.is_contiguous():
+        raise ValueError("retention: decay is fp32 [heads]")
+    if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (heads, dk, dv):
+        raise ValueError("retention: state is contiguous fp32 [slots, heads, dk, dv]")
+    if step.num_tokens != n:
+        raise ValueError("retention: the step describes another number of tokens")
+    if not retention_supported(dk, dv):
+        raise ValueError(f"retention: head geometry {dk} x {dv} is not served (dk <= 256)")
+    if half < 0 or 2 * half > dk or (half and (rot_table is None or rot_table.dtype != torch.float32 or rot_table.dim() != 2
+                                               or rot_table.shape[0] != n or rot_table.shape[1] < 2 * half
+                                               or not rot_table.is_contiguous())):
+        raise ValueError("retention: the rotation table is what rotation_table() returns for this step and these pairs")
+    if out is None:
+        out = torch.empty(n, heads * dv, dtype=st, device=q.device)
+    elif out.dtype != st or tuple(out.shape) != (n, heads * dv) or out.stride(1) != 1:
+        raise ValueError("retention: out is [n, heads dv] in the storage dtype with a unit inner stride")
+    ld = lambda t: max(t.stride(0), t.shape[1])  # noqa: E731  (one row: its stride means nothing)
+    decode = step.longest_run == 1
+    o = None if decode else torch.empty(n, heads * dv, dtype=torch.float32, device=q.device)
+    L.check(L.lib().ll_retention(q.data_ptr(), ld(q), k.data_ptr(), ld(k), v.data_ptr(), ld(v), heads, dk, dv, L.ptr(rot_table) if half else 0,
+                                 rot_table.shape[1] if half else 0, int(half), float(k_scale), decay.data_ptr(), step.seq_start.data_ptr(),
+                                 step.seq_first_pos.data_ptr(), step.seq_slot.data_ptr(), state.data_ptr(), L.ptr(o), gate.data_ptr(), ld(gate),
+                                 float(eps), out.data_ptr(), ld(out), n, step.num_seqs, L.dtype_code(st), L.stream_ptr()), "retention")
+    if not decode:
+        gated_out_norm(o, None, eps, parts=heads, gate=gate, gate_kind="silu", out=out)
+    return out
+
+
 _GATES = {None: 0, "silu": 1, "sigmoid": 2}
 
 

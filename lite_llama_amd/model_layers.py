@@ -35,6 +35,11 @@ description, out of mixers that take a ragged step (executor/ragged.py) and keep
                                a low-rank projection, a state that is corrected towards the token's value (kernels/recurrent.py)
   * :class:`RealGatedLRU`      a per-channel recurrence behind a convolution whose two gates are block-diagonal products, times a
                                gelu branch (kernels/recurrent.py)
+  * :class:`GatedWindowAttention`  a rotation of entry pairs, a window that keeps a sequence's first keys, a learned sink, one sigmoid gate
+                               per head; keys and values are its own or those another layer has cached (kernels/attention.py)
+  * :class:`Retention`         linear attention with a fixed decay per head over rotated queries and keys, heads normed without a
+                               weight, a silu gate (kernels/recurrent.py)
+  * :class:`GroupSoftmaxMoE`   softmax scores over all experts, the groups with the best members stay, chosen scores renormalised
   * :class:`SquareMoE`         sigmoid scores that multiply the experts' inputs (not renormalised), experts ``down(relu(up h)^2)``, a
                                shared expert of the same form with a per-token scale
 
@@ -44,7 +49,8 @@ kernels/norm_act.py::gated_group_norm for layers that wrap each sublayer in two 
 Projections run through the framework's linear layers (library GEMM for unquantised weights), with everything that reads one
 input fused into one launch at load time.  Families: Rakevik (``"architecture": "Rakevik"``: :class:`MixerLayer`),
 Rukedra (:class:`SandwichLayer`), Fekanex (:class:`ParallelLayer`: one norm per layer, mixer and feed-forward read its
-output side by side, and -- with a dense feed-forward -- share ONE input projection and ONE output projection), Nivotar
+output side by side, and -- with a dense feed-forward or a shared expert -- share ONE input projection and ONE output
+projection), Kokuvik (the same layer with other mixers and feed-forwards), Nivotar
 (:class:`PostNormLayer`: sublayers read the residual stream itself, the norm sits on each sublayer's result) and Tusasun
 (:class:`StreamLayer`: several residual streams that every sublayer reads, mixes and writes through learned vectors).
 """
@@ -67,7 +73,8 @@ from .kernels.attention import (conv_rope_cache, latent_kv_prep, qk_norm_cache, 
 from .kernels.fused_moe import group_router, sparse_glu_experts, sparse_square_experts
 from .kernels.norm_act import (GatedUpdate, StreamUpdate, SummedUpdate, add_rmsnorm_shift, cast_pair, embed_pair, gated_group_norm,
                                glu_act, relu_square, residual_set, softcap_, stream_norm)
-from .kernels.recurrent import (conv_act, delta_scan, gated_linear_scan, gated_out_norm, linear_scan, mingru_scan, rglru_scan)
+from .kernels.recurrent import (conv_act, delta_scan, gated_linear_scan, gated_out_norm, linear_scan, mingru_scan, retention,
+                                rglru_scan)
 from .linear import ReplicatedLinear
 
 
@@ -76,14 +83,17 @@ from .linear import ReplicatedLinear
 # ------------------------------------------------------------------------------------- #
 @dataclass(frozen=True)
 class RotarySpec:
-    """Rotation of entry pairs (2i, 2i + 1) of the first ``dims`` entries by ``position * f_i``, ``f_i = base^(-2i / dims)``;
-    with ``factor`` the frequencies are rescaled between a fast and a slow end (YaRN)."""
+    """Rotation of the first ``dims`` entries in pairs by ``position * f_i``, ``f_i = base^(-2i / dims)``; with ``factor`` the
+    frequencies are rescaled, either between a fast and a slow end (YaRN) or -- ``high > 0`` -- by bands of wavelength: kept below
+    ``original / high``, divided by ``factor`` above ``original / low``, blended in between."""
     dims: int
     base: float
     factor: float = 0.0         # 0: no scaling
     original: float = 0.0       # positions the unscaled frequencies were made for
     fast: float = 0.0           # turns over `original` positions above which a pair keeps its frequency
     slow: float = 0.0           # ... and below which it is divided by `factor`
+    low: float = 0.0            # bands: turns over `original` positions below which a pair is divided by `factor`
+    high: float = 0.0           # ... and above which it keeps its frequency
 
     def table(self) -> tuple[list[float], float]:
         """``(frequency per pair, amplitude of cos / sin)``."""
@@ -91,6 +101,8 @@ class RotarySpec:
         f = [self.base ** (-2.0 * i / self.dims) for i in range(half)]
         if not self.factor:
             return f, 1.0
+        if self.high:
+            return [self._banded(fi) for fi in f], 1.0
 
         def pair_of(turns: float) -> float:   # the (fractional) pair that makes `turns` turns over `original` positions
             return self.dims * math.log(self.original / (2 * math.pi * turns)) / (2 * math.log(self.base))
@@ -103,11 +115,26 @@ class RotarySpec:
             out.append(fi / self.factor * ramp + fi * (1.0 - ramp))
         return out, 0.1 * math.log(self.factor) + 1.0
 
+    def _banded(self, f: float) -> float:
+        wavelength = 2 * math.pi / f
+        if wavelength < self.original / self.high:
+            return f
+        if wavelength > self.original / self.low:
+            return f / self.factor
+        s = (self.original / wavelength - self.low) / (self.high - self.low)
+        return (1 - s) * f / self.factor + s * f
+
     @staticmethod
     def from_config(rot: Mapping) -> "RotarySpec":
         sc = rot.get("scaling")
         if not sc:
             return RotarySpec(int(rot["dims"]), float(rot["base"]))
+        if "high" in sc:
+            spec = RotarySpec(int(rot["dims"]), float(rot["base"]), float(sc["factor"]), float(sc["original"]), low=float(sc["low"]),
+                              high=float(sc["high"]))
+            if not (spec.factor > 0 and spec.original > 0 and 0 < spec.low < spec.high):
+                raise ValueError(f"wavelength bands {spec.low} .. {spec.high} over {spec.original} positions, factor {spec.factor}")
+            return spec
         return RotarySpec(int(rot["dims"]), float(rot["base"]), float(sc["factor"]), float(sc["original"]), float(sc["fast"]),
                           float(sc["slow"]))
 
@@ -136,7 +163,7 @@ class StateSpaceSpec:
 @dataclass(frozen=True)
 class MixerSpec:
     kind: str                   # "attention" | "hgrn2" | "latent_attention" | "mingru" | "conv_attention" | "attention_ssd" | "decay_linear" | "gla"
-                                # | "distance_attention" | "channel_delta" | "rglru"
+                                # | "distance_attention" | "channel_delta" | "rglru" | "window_attention" | "retention"
     heads: int = 1
     dim: int = 0                # per-head query / key width (latent attention: the unrotated part)
     vdim: int = 0               # per-head value width
@@ -147,8 +174,9 @@ class MixerSpec:
     rot_dim: int = 0            # latent attention: rotated query / key entries per head (the key's are shared by all heads)
     kv_rank: int = 0            # latent attention: width of the cached key/value latent
     q_rank: int = 0             # latent attention: width of the query latent (0: queries are projected directly)
-    window: int = 0             # latent / conv attention: 0 = causal, else the last `window` positions are seen
-    keep_first: int = 0         # conv attention: with a window, the sequence's first positions that stay visible
+    window: int = 0             # latent / conv / window attention: 0 = causal, else the last `window` positions are seen
+    keep_first: int = 0         # conv / window attention: with a window, the sequence's first positions that stay visible
+    kv_from: int | None = None  # window attention: the layer whose cached keys and values this one reads (None: its own)
     bias: bool = False          # conv attention: q / k / v projections carry a bias
     conv_taps: int = 0          # conv attention, channel_delta, rglru: taps of the causal convolution over time behind the projections (0: none)
     unit_norm: bool = False     # conv attention: q / k heads divided by their root mean square (no weight) after the rotation
@@ -160,7 +188,7 @@ class MixerSpec:
     blocks: int = 1             # rglru: equal parts of the channels with gate matrices of their own
     ssd: StateSpaceSpec | None = None           # attention_ssd: the state-space branch beside the attention
     branch_scales: tuple = (1.0, 1.0)           # attention_ssd: result = scales[0] * attention + scales[1] * state-space
-    decay: tuple = ()           # decay_linear: the fixed decay of every head
+    decay: tuple = ()           # decay_linear, retention: the fixed decay of every head
     tau: float = 1.0            # gla: decay = sigmoid(.)^(1 / tau)
     decay_rank: int = 0         # gla, channel_delta: width of the low-rank projection in front of the decay logits
     gate_rank: int = 0          # channel_delta: width of the low-rank projection in front of the output gate
@@ -173,11 +201,12 @@ class MixerSpec:
 class MlpSpec:
     kind: str = "dense"         # "dense" | "moe"
     ff: int = 0                 # dense: hidden width; moe: hidden width of one expert
-    act: str = "xielu"          # dense: "xielu" (up / down) | "gelu_tanh" | "clamped" | "silu" (gate / up / down); moe: also "relu_square" (up / down)
+    act: str = "xielu"          # dense: "xielu" (up / down) | "gelu_tanh" | "clamped" | "silu" (gate / up / down); dense, moe: "relu_square" (up / down)
     limit: float = 0.0          # "clamped": gate <= limit, |up| <= limit
     scoring: str = "sigmoid"    # moe: "sigmoid" (scores over groups) | "softmax_chosen" (largest logits, softmax over them)
                                 # | "softmax_all" (softmax over all outputs, chosen by score + correction)
                                 # | "sigmoid_plain" (sigmoid scores, not renormalised)
+                                # | "softmax_groups" (softmax over all outputs, groups by their best member, renormalised)
     identity: int = 0           # moe, "softmax_all": router outputs beyond `experts` that stand for the input itself
     bias: bool = False          # dense: every projection carries a bias
     experts: int = 0
@@ -249,6 +278,8 @@ class LayeredGeometry:
             return _rukedra_geometry(config, name)
         if name == "fekanex":
             return _fekanex_geometry(config, name)
+        if name == "kokuvik":
+            return _kokuvik_geometry(config, name)
         layers = []
         for entry in config["layers"]:
             m, kind = entry["mixer"], entry["type"]
@@ -488,17 +519,106 @@ def _tusasun_geometry(config: Mapping, name: str, shapes: Mapping) -> LayeredGeo
                            streams=streams, norm_base=1.0)
 
 
+def _kokuvik_geometry(config: Mapping, name: str) -> LayeredGeometry:
+    """Kokuvik: per layer one of two mixers -- ``retention`` (linear attention with a fixed decay per head over rotated queries and
+    keys), ``attention`` (rotated, windowed, with kept first keys, a learned sink and a gate per head; it may read the keys and
+    values an earlier attention layer has cached) --, beside it, under the same norm, a dense squared-relu feed-forward with
+    biases or grouped softmax experts with a shared one; an output head of its own."""
+    layers = []
+    for index, entry in enumerate(config["layers"]):
+        m, kind = entry["mixer"], entry["type"]
+        if kind == "attention":
+            rot = RotarySpec.from_config(m["rot"]) if m.get("rot") else None
+            mask = m.get("mask") or {}
+            source = m.get("kv_from")
+            spec = MixerSpec("window_attention", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             kv_heads=int(m.get("kv_heads") or m["heads"]), scale=float(m["scale"]), rotary=rot,
+                             window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0),
+                             kv_from=None if source is None else int(source))
+            if spec.heads % spec.kv_heads:
+                raise ValueError(f"layer {index}: {spec.heads} query heads do not divide over {spec.kv_heads} key/value heads")
+            if spec.kv_from is not None:
+                owner = layers[spec.kv_from].mixer if 0 <= spec.kv_from < index else None
+                if owner is None or owner.kind != spec.kind or owner.kv_from is not None:
+                    raise ValueError(f"layer {index} reads the keys and values of layer {spec.kv_from}, which is not an earlier attention "
+                                     "layer with its own")
+                if (owner.kv_heads, owner.dim, owner.vdim) != (spec.kv_heads, spec.dim, spec.vdim) or owner.rotary != spec.rotary:
+                    raise ValueError(f"layer {index} reads the keys and values of layer {spec.kv_from}, whose heads or rotation differ")
+        elif kind == "retention":
+            rot = RotarySpec(int(m["rot"]["dims"]), float(m["rot"]["base"])) if m.get("rot") else None
+            spec = MixerSpec("retention", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), rotary=rot,
+                             decay=tuple(float(d) for d in m["decay"]))
+            if len(spec.decay) != spec.heads:
+                raise ValueError(f"layer {index}: {len(spec.decay)} decays for {spec.heads} heads")
+        else:
+            raise ValueError(f"unsupported mixer type {kind!r}; supported: retention, attention")
+        if rot is not None and (rot.dims > spec.dim or rot.dims % 2):
+            raise ValueError(f"layer {index}: {rot.dims} rotated entries do not fit heads of {spec.dim}")
+        mlp = entry.get("mlp")
+        if mlp is None:
+            mspec = None
+        elif mlp.get("kind", "dense") == "dense":
+            mspec = MlpSpec("dense", ff=int(mlp["ff"]), act="relu_square", bias=True)
+        elif mlp["kind"] == "moe":
+            r = mlp["router"]
+            groups = r.get("groups") or {}
+            mspec = MlpSpec("moe", ff=int(mlp["expert"]["ff"]), act="silu", experts=int(r["experts"]), top=int(r["top"]),
+                            scoring="softmax_groups", group_count=int(groups.get("count", 1)), group_keep=int(groups.get("keep", 1)),
+                            shared_ff=int((mlp.get("shared") or {}).get("ff", 0)))
+            if mspec.group_count < 1 or mspec.experts % mspec.group_count or not 1 <= mspec.group_keep <= mspec.group_count \
+                    or not 1 <= mspec.top <= mspec.group_keep * (mspec.experts // mspec.group_count):
+                raise ValueError(f"layer {index}: {mspec.top} of {mspec.experts} experts cannot be chosen from "
+                                 f"{mspec.group_keep} of {mspec.group_count} groups")
+        else:
+            raise ValueError(f"unsupported feed-forward kind {mlp.get('kind')!r}; supported: dense, moe")
+        layers.append(LayerSpec(spec, ff=mspec.ff if mspec else 0, mlp_kind=mspec.kind if mspec else "dense", mlp=mspec))
+    return LayeredGeometry(name=name, vocab_size=int(config["vocab"]), width=int(config["width"]), eps=float(config["norm"]["eps"]),
+                           layers=tuple(layers), token_shift=False, parallel=True)
+
+
+def _aligned(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
 def _linear(inp: int, out: int) -> ReplicatedLinear:
     return ReplicatedLinear(inp, out)
 
 
-def _padded_linear(inp: int, out: int, used_rows: int) -> ReplicatedLinear:
+def _padded_linear(inp: int, out: int, used_rows: int, bias_rows: int = 0) -> ReplicatedLinear:
     """A projection fused from members that start on 16-byte borders: ``out`` rows of which the members fill ``used_rows``, the rest
-    are zeros that no checkpoint tensor fills."""
-    lin = ReplicatedLinear(inp, out)
+    are zeros that no checkpoint tensor fills.  ``bias_rows``: how many rows belong to members with a bias (0: there is none)."""
+    lin = ReplicatedLinear(inp, out, bias=bias_rows > 0)
     lin.weight.data.zero_()
     lin.weight.ll_unfilled = (out - used_rows) * inp
+    if bias_rows:
+        lin.bias.data.zero_()
+        lin.bias.ll_unfilled = out - bias_rows
     return lin
+
+
+class StepRotation:
+    """The rotation of a mixer's q / k heads: frequencies on the device of the first step (fp32, not a buffer: a module-wide cast must
+    not touch the angles), cos / sin per token once per step for all layers that rotate alike."""
+
+    def __init__(self, spec: RotarySpec | None):
+        self.values, self.amp = spec.table() if spec is not None else ([], 1.0)
+        self.pairs = len(self.values)
+        self.freq = None
+        self._key = ("rotation", self.pairs, self.amp, tuple(self.values))
+
+    def table(self, step, device):
+        """:func:`rotation_table` of the step (``None`` without rotated pairs)."""
+        if not self.pairs:
+            return None
+        if self.freq is None or self.freq.device != device:
+            self.freq = torch.tensor(self.values, dtype=torch.float64).to(torch.float32).to(device)
+        shared = getattr(step, "shared", None)
+        table = shared.get(self._key) if shared is not None else None
+        if table is None:
+            table = rotation_table(step, self.freq, self.pairs, self.amp)
+            if shared is not None:
+                shared[self._key] = table
+        return table
 
 
 def _vector(n: int) -> nn.Parameter:
@@ -746,9 +866,7 @@ class ConvRotaryAttention(nn.Module):
         self.conv_weight = (nn.Parameter(torch.zeros(self.channels, s.conv_taps, dtype=torch.float16), requires_grad=False)
                             if s.conv_taps else None)
         self.value_blend = _vector(1) if s.value_mix else None
-        self._freq_values, self.amp = s.rotary.table() if s.rotary is not None else ([], 1.0)
-        self.pairs = len(self._freq_values)
-        self._freq = None   # fp32 on the device of the first step (not a buffer: a module-wide cast must not touch the angles)
+        self.rotation = StepRotation(s.rotary)
         self._sink = None   # zeros [heads]: exp(0) = 1 in every denominator
 
     def cache_run(self) -> dict:
@@ -760,23 +878,13 @@ class ConvRotaryAttention(nn.Module):
         s = self.spec
         rows = self.in_proj(h)
         k_cache, v_cache = cache.kv_buffer[run]
-        if self.pairs and (self._freq is None or self._freq.device != h.device):
-            self._freq = torch.tensor(self._freq_values, dtype=torch.float64).to(torch.float32).to(h.device)
         if s.unit_sink and (self._sink is None or self._sink.device != h.device or self._sink.dtype != h.dtype):
             self._sink = torch.zeros(s.heads, dtype=h.dtype, device=h.device)
         source = cache.value_source[run]
-        table = None
-        if self.pairs:   # cos / sin per token: once per step for all layers that rotate alike
-            key = ("rotation", self.pairs, self.amp, tuple(self._freq_values))
-            shared = getattr(step, "shared", None)
-            table = shared.get(key) if shared is not None else None
-            if table is None:
-                table = rotation_table(step, self._freq, self.pairs, self.amp)
-                if shared is not None:
-                    shared[key] = table
+        table = self.rotation.table(step, h.device)
         q = conv_rope_cache(rows, s.heads, s.kv_heads, s.dim, s.vdim, step, k_cache, v_cache, bias=self.qkv_bias,
-                            conv_weight=self.conv_weight, conv_state=cache.conv[run], freq=self._freq, pairs=self.pairs,
-                            amp=self.amp, unit_norm=s.unit_norm, eps=self.eps,
+                            conv_weight=self.conv_weight, conv_state=cache.conv[run], freq=self.rotation.freq, pairs=self.rotation.pairs,
+                            amp=self.rotation.amp, unit_norm=s.unit_norm, eps=self.eps,
                             v_source=cache.kv_buffer[source][1] if source is not None else None,
                             v_blend=self.value_blend if source is not None else None, rot_table=table)
         o = ragged_attention(q, k_cache, v_cache, s.scale, step, token_table, sink=self._sink if s.unit_sink else None,
@@ -799,6 +907,56 @@ class ChosenSoftmaxMoE(nn.Module):
     def forward(self, h):
         ids, weights, _ = group_router(h, self.router_weight, self.spec.top, scoring=self.spec.scoring)
         return sparse_glu_experts(h, self.gate_up_weight, self.down_weight, ids, weights)
+
+
+class GroupSoftmaxMoE(ChosenSoftmaxMoE):
+    """Scores are the softmax (fp32) over all router outputs; the experts form equal groups of neighbours, a group scores as its
+    best member, the best groups stay eligible; the ``top`` best eligible experts weigh in with their scores divided by the
+    scores' sum.  A shared expert is the layer's: it rides in the layer's two projections."""
+
+    def forward(self, h):
+        s = self.spec
+        ids, weights, _ = group_router(h, self.router_weight, s.top, s.group_count, s.group_keep, scoring=s.scoring)
+        return sparse_glu_experts(h, self.gate_up_weight, self.down_weight, ids, weights)
+
+
+class GatedWindowAttention(nn.Module):
+    """``q | k | v | the layer's columns | g`` in one projection (the last two on 16-byte borders); rotation and cache write in one
+    launch; attention over the paged cache with a window, kept first keys, a learned sink and one sigmoid gate per head in one
+    launch.  With ``kv_from`` the projection has no ``k | v`` and attention reads the keys (as that layer's cache holds them,
+    rotated) and values of another layer.  The heads' outputs go to ``out`` (a column range of the layer's output projection input):
+    the output projection is the layer's."""
+
+    def __init__(self, width: int, spec: MixerSpec, eps: float, extra: int = 0, extra_bias: bool = False):
+        super().__init__()
+        self.spec, self.extra = spec, extra
+        s = spec
+        self.kv_heads = s.kv_heads if s.kv_from is None else 0      # key/value heads this layer projects and caches
+        self.channels = (s.heads + self.kv_heads) * s.dim + self.kv_heads * s.vdim
+        self.extra_off = _aligned(self.channels)
+        self.gate_off = _aligned(self.extra_off + extra)
+        self.in_proj = _padded_linear(width, _aligned(self.gate_off + s.heads), self.channels + extra + s.heads,
+                                      bias_rows=extra if extra_bias else 0)
+        self.sink = _vector(s.heads)
+        self.rotation = StepRotation(s.rotary)
+
+    def cache_run(self) -> dict:
+        s = self.spec
+        if s.kv_from is not None:
+            return {"kind": "shared", "source": s.kv_from}
+        return {"kind": "attention", "kv_heads": s.kv_heads, "dk": s.dim, "dv": s.vdim}
+
+    def forward(self, h, step, cache, run: int, token_table, out=None):
+        s = self.spec
+        rows = self.in_proj(h)
+        k_cache, v_cache = cache.kv_buffer[run]
+        table = self.rotation.table(step, h.device)
+        own = self.kv_heads > 0
+        q = conv_rope_cache(rows, s.heads, self.kv_heads, s.dim, s.vdim, step, k_cache if own else None, v_cache if own else None,
+                            freq=self.rotation.freq, pairs=self.rotation.pairs, amp=self.rotation.amp, rot_table=table)
+        o = ragged_attention(q, k_cache, v_cache, s.scale, step, token_table, sink=self.sink, window=s.window, keep_first=s.keep_first,
+                             head_gate=rows[:, self.gate_off:self.gate_off + s.heads], out=out)
+        return o, (rows[:, self.extra_off:self.extra_off + self.extra] if self.extra else None)
 
 
 class WindowAttentionSSD(nn.Module):
@@ -880,6 +1038,40 @@ class DecayLinearAttention(nn.Module):
         o = linear_scan(rows[:, :qk], rows[:, qk:2 * qk], rows[:, 2 * qk:2 * qk + v], s.heads, s.dim, s.vdim, step,
                         cache.recurrent[run], act=True, head_decay=self._decay)
         return self.o_proj(gated_out_norm(o, self.out_norm_weight, self.eps, gate=rows[:, 2 * qk + v:], gate_kind="sigmoid"))
+
+
+class Retention(nn.Module):
+    """``q | k | v | g | the layer's columns`` in one projection (members on 16-byte borders); per head, over rotated q and k with k
+    times ``dim^(-1/2)``, ``S <- decay_h S + k v^T``, ``o = S^T q`` over the fp32 state slots; every head divided by its root mean square,
+    times ``silu(g)``.  The result goes to ``out`` (a column range of the layer's output projection input): the output projection is
+    the layer's."""
+
+    def __init__(self, width: int, spec: MixerSpec, eps: float, extra: int = 0, extra_bias: bool = False):
+        super().__init__()
+        self.spec, self.eps, self.extra = spec, eps, extra
+        self.qk, self.v = spec.heads * spec.dim, spec.heads * spec.vdim
+        self.k_off = _aligned(self.qk)
+        self.v_off = _aligned(self.k_off + self.qk)
+        self.g_off = _aligned(self.v_off + self.v)
+        self.extra_off = _aligned(self.g_off + self.v)
+        self.in_proj = _padded_linear(width, _aligned(self.extra_off + extra), 2 * (self.qk + self.v) + extra,
+                                      bias_rows=extra if extra_bias else 0)
+        self.rotation = StepRotation(spec.rotary)
+        self._decay = None   # fp32 on the device of the first step (not a buffer: a module-wide cast must not round the decays)
+
+    def cache_run(self) -> dict:
+        return {"kind": "recurrent", "heads": self.spec.heads, "dk": self.spec.dim, "dv": self.spec.vdim}
+
+    def forward(self, h, step, cache, run: int, token_table, out=None):
+        s = self.spec
+        rows = self.in_proj(h)
+        if self._decay is None or self._decay.device != h.device:
+            self._decay = torch.tensor(s.decay, dtype=torch.float64).to(torch.float32).to(h.device)
+        part = lambda at, count: rows[:, at:at + count]  # noqa: E731
+        o = retention(part(0, self.qk), part(self.k_off, self.qk), part(self.v_off, self.v), s.heads, s.dim, s.vdim, step,
+                      cache.recurrent[run], decay=self._decay, gate=part(self.g_off, self.v), eps=self.eps, k_scale=s.dim ** -0.5,
+                      half=self.rotation.pairs, rot_table=self.rotation.table(step, h.device), out=out)
+        return o, (part(self.extra_off, self.extra) if self.extra else None)
 
 
 class GatedLinearAttention(nn.Module):
@@ -988,10 +1180,6 @@ class BiasedDistanceAttention(nn.Module):
         q = qk_norm_cache(self.in_proj(h), s.heads, s.kv_heads, s.dim, s.vdim, self.q_norm_weight, self.k_norm_weight, self.eps, 0.0, 1,
                           step, k_cache, v_cache)
         return self.o_proj(ragged_attention(q, k_cache, v_cache, s.scale, step, token_table, cap=s.softcap, dist_bias=self._by_distance))
-
-
-def _aligned(n: int) -> int:
-    return (n + 7) // 8 * 8
 
 
 class ChannelDeltaMixer(nn.Module):
@@ -1104,7 +1292,7 @@ class SquareMoE(nn.Module):
 MIXERS = {"attention": SinkAttention, "hgrn2": GatedLinearMixer, "latent_attention": LatentAttention, "mingru": MinGRU,
           "conv_attention": ConvRotaryAttention, "attention_ssd": WindowAttentionSSD, "decay_linear": DecayLinearAttention,
           "gla": GatedLinearAttention, "distance_attention": BiasedDistanceAttention, "channel_delta": ChannelDeltaMixer,
-          "rglru": RealGatedLRU}
+          "rglru": RealGatedLRU, "window_attention": GatedWindowAttention, "retention": Retention}
 
 
 class MixerLayer(nn.Module):
@@ -1159,10 +1347,11 @@ class SandwichLayer(nn.Module):
 
 
 class ParallelLayer(nn.Module):
-    """``x <- x + (mixer(h) + feed_forward(h))`` with ``h = norm(x)``: one norm, both sublayers read it.  With a dense
-    feed-forward, ``q | k | v | gate | up`` are ONE input projection and ``[heads' outputs | activation]`` go through ONE output
-    projection ``[W_o | W_down]``, whose fp32 accumulation is the sum of the two sublayers.  With experts, the mixer's output
-    projection gives one row and the experts' slots ride beside it as a :class:`SummedUpdate` into the next norm launch."""
+    """``x <- x + (mixer(h) + feed_forward(h))`` with ``h = norm(x)``: one norm, both sublayers read it.  What every token runs of the
+    feed-forward -- a dense one, or the shared expert beside routed ones -- joins the mixer: its first products are columns of
+    the mixer's ONE input projection, and ``[heads' outputs | activation]`` go through ONE output projection ``[W_o | W_down]``, whose
+    fp32 accumulation is the sum of the two (their biases are its bias).  Routed experts' slots ride beside that row as a
+    :class:`SummedUpdate` into the next norm launch."""
 
     slope = 1.702   # inside the sigmoid of the clamped GLU
 
@@ -1171,21 +1360,32 @@ class ParallelLayer(nn.Module):
         self.eps = geo.eps
         w, m = geo.width, spec.mixer
         self.norm1_weight = _vector(w)
-        self.dense = spec.mlp if (spec.mlp is not None and spec.mlp.kind == "dense") else None
-        ff = self.dense.ff if self.dense is not None else 0
-        self.mixer = MIXERS[m.kind](w, m, geo.eps, extra=2 * ff)
+        mlp = spec.mlp
+        # the feed-forward's part in the two projections: hidden width, activation, columns of the input projection
+        if mlp is None:
+            self.ff, self.act, biased = 0, "", False
+        elif mlp.kind == "dense":
+            self.ff, self.act, biased = mlp.ff, mlp.act, mlp.bias
+        else:
+            self.ff, self.act, biased = mlp.shared_ff, mlp.act, False
+        self.limit = mlp.limit if mlp is not None else 0.0
+        self.in_cols = self.ff * (1 if self.act == "relu_square" else 2)
+        self.mixer = MIXERS[m.kind](w, m, geo.eps, extra=self.in_cols, **({"extra_bias": True} if biased else {}))
         self.heads_width = m.heads * m.vdim
-        self.out_proj = _linear(self.heads_width + ff, w)
-        self.experts = ChosenSoftmaxMoE(w, spec.mlp) if (spec.mlp is not None and spec.mlp.kind == "moe") else None
+        self.out_proj = ReplicatedLinear(self.heads_width + self.ff, w, bias=biased)
+        self.experts = None
+        if mlp is not None and mlp.kind == "moe":
+            self.experts = (GroupSoftmaxMoE if mlp.scoring == "softmax_groups" else ChosenSoftmaxMoE)(w, mlp)
 
     def forward(self, x, pending, step, cache, run: int, token_table):
         """``(x, pending)``: the fp32 residual (updated in place) and the update still to enter it.  Returns the same pair."""
         h, x = add_rmsnorm_shift(x, pending, self.norm1_weight, self.eps, x_out=x)
-        ff = self.dense.ff if self.dense is not None else 0
-        mixed = torch.empty(h.shape[0], self.heads_width + ff, dtype=h.dtype, device=h.device)
-        _, gate_up = self.mixer(h, step, cache, run, token_table, out=mixed[:, :self.heads_width])
-        if ff:
-            glu_act(gate_up, ff, self.dense.act, limit=self.dense.limit, slope=self.slope, out=mixed[:, self.heads_width:])
+        mixed = torch.empty(h.shape[0], self.heads_width + self.ff, dtype=h.dtype, device=h.device)
+        _, hidden = self.mixer(h, step, cache, run, token_table, out=mixed[:, :self.heads_width])
+        if self.ff and self.act == "relu_square":
+            relu_square(hidden, self.ff, out=mixed[:, self.heads_width:])
+        elif self.ff:
+            glu_act(hidden, self.ff, self.act, limit=self.limit, slope=self.slope, out=mixed[:, self.heads_width:])
         row = self.out_proj(mixed)
         return x, SummedUpdate(row, self.experts(h) if self.experts is not None else None)
 

@@ -716,6 +716,67 @@ def _fekanex_translator(geo) -> Translator:
     return translate
 
 
+def _kokuvik_translator(geo, layers) -> Translator:
+    """Tensor names of a Kokuvik checkpoint -> parameters of :class:`lite_llama_amd.model_layers.LayeredLM` built from
+    :class:`ParallelLayer`: everything that reads a layer's normed input -- ``mix.q / k / v / g`` and the first products of the dense
+    feed-forward (``mlp.up``, with its bias) or of the shared expert (``mlp.shared.gate / up``) -- lands in its row range of the
+    layer's one input projection (``layers``: the model's layers know where their members lie); ``mix.o`` and ``mlp.down`` (or
+    ``mlp.shared.down``) in their COLUMN ranges of the one output projection; routed experts ``mlp.e<k>.*`` in the stacked expert
+    tensors."""
+    fixed = {"embed": "embed_tokens.weight", "final.norm": "norm_weight", "head": "lm_head.weight"}
+    plain = {"norm1": "norm1_weight", "mix.sink": "mixer.sink", "mlp.router": "experts.router_weight"}
+    expert_leaf = re.compile(r"^mlp\.e(\d+)\.(gate|up|down)$")
+
+    def fused(layer, spec):
+        """``{checkpoint leaf: (parameter, Region)}`` of one layer."""
+        m, x, out = spec.mixer, layer.mixer, {}
+
+        def rows(param, *members):
+            for leaf, first, count in members:
+                out[leaf] = (param, Region(rows=(first, count)))
+
+        weight = "mixer.in_proj.weight"
+        if m.kind == "retention":
+            rows(weight, ("mix.q", 0, x.qk), ("mix.k", x.k_off, x.qk), ("mix.v", x.v_off, x.v), ("mix.g", x.g_off, x.v))
+        else:
+            q, k, v = m.heads * m.dim, x.kv_heads * m.dim, x.kv_heads * m.vdim
+            rows(weight, ("mix.q", 0, q), ("mix.g", x.gate_off, m.heads))
+            if x.kv_heads:
+                rows(weight, ("mix.k", q, k), ("mix.v", q + k, v))
+        out["mix.o"] = ("out_proj.weight", Region(cols=(0, layer.heads_width)))
+        if layer.ff and spec.mlp.kind == "dense":
+            rows(weight, ("mlp.up", x.extra_off, layer.ff))
+            rows("mixer.in_proj.bias", ("mlp.up.b", x.extra_off, layer.ff))
+            out["mlp.down"] = ("out_proj.weight", Region(cols=(layer.heads_width, layer.ff)))
+            out["mlp.down.b"] = ("out_proj.bias", whole)
+        elif layer.ff:
+            rows(weight, ("mlp.shared.gate", x.extra_off, layer.ff), ("mlp.shared.up", x.extra_off + layer.ff, layer.ff))
+            out["mlp.shared.down"] = ("out_proj.weight", Region(cols=(layer.heads_width, layer.ff)))
+        return out
+
+    members = [fused(layer, spec) for layer, spec in zip(layers, geo.layers)]
+
+    def translate(key: str) -> Target:
+        if key in fixed:
+            return fixed[key], whole
+        m = re.match(r"^l(\d+)\.(.+)$", key)
+        if m is None or int(m.group(1)) >= len(geo.layers):
+            return key, whole  # unknown: load_weights reports it
+        index, leaf = int(m.group(1)), m.group(2)
+        if leaf in members[index]:
+            name, region = members[index][leaf]
+            return f"layers.{index}.{name}", region
+        e = expert_leaf.match(leaf)
+        if e is not None:
+            k, proj = int(e.group(1)), e.group(2)
+            if proj == "down":
+                return f"layers.{index}.experts.down_weight", expert(k)
+            return f"layers.{index}.experts.gate_up_weight", expert_half(k, 0 if proj == "gate" else 1)
+        return f"layers.{index}.{plain.get(leaf, leaf)}", whole
+
+    return translate
+
+
 def _nivotar_translator(geo) -> Translator:
     """Tensor names of a Nivotar checkpoint -> parameters of :class:`lite_llama_amd.model_layers.LayeredLM` built from
     :class:`PostNormLayer`.  Everything that reads a mixer's input lands in its row range of the mixer's ONE input projection
@@ -872,7 +933,8 @@ def _load_layered(config: Mapping, checkpoints_dir, device, dtype=None, **_):
     geo = LayeredGeometry.from_config(config, name=family,
                                       shapes=tensor_shapes(checkpoints_dir) if family in ("nivotar", "tusasun") else None)
     model = LayeredLM(geo, dtype=dtype or torch.bfloat16).to(device)
-    translator = (_rukedra_translator(geo) if geo.sandwich else _fekanex_translator(geo) if geo.parallel
+    translator = (_rukedra_translator(geo) if geo.sandwich else _kokuvik_translator(geo, model.layers) if family == "kokuvik"
+                  else _fekanex_translator(geo) if geo.parallel
                   else _nivotar_translator(geo) if geo.post_norm else _tusasun_translator(geo, model.layers) if geo.streams
                   else _layered_translator(geo))
     with torch.no_grad():
@@ -881,7 +943,7 @@ def _load_layered(config: Mapping, checkpoints_dir, device, dtype=None, **_):
 
 
 MODEL_FAMILIES: dict[str, Callable] = {"rakevik": _load_layered, "rukedra": _load_layered, "fekanex": _load_layered,
-                                       "nivotar": _load_layered, "tusasun": _load_layered}
+                                       "nivotar": _load_layered, "tusasun": _load_layered, "kokuvik": _load_layered}
 
 
 def load_pretrained(checkpoints_dir: str | Path, *, device: str | torch.device = "cuda", quantization: str | None = None,
