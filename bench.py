@@ -120,6 +120,13 @@ def parse():
                          "--layered-dtype picks the dtype")
     ap.add_argument("--tusasun-sizes", default="compact,wide", help="which size points of benchmarks/tusasun_bench.py::SIZES to run")
     ap.add_argument("--tusasun-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
+    ap.add_argument("--kokuvik", action="store_true",
+                    help="instead of the headline: prefill / decode throughput and per-kernel roofline fractions of the Kokuvik design "
+                         "(retention, windowed attention with kept first keys, a learned sink, a gate per head and shared keys / values, "
+                         "squared-relu and grouped-softmax expert feed-forwards) beside the closest models of the layered family "
+                         "(benchmarks/kokuvik_bench.py); --layered-dtype picks the dtype")
+    ap.add_argument("--kokuvik-sizes", default="compact,wide", help="which size points of benchmarks/kokuvik_bench.py::SIZES to run")
+    ap.add_argument("--kokuvik-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
     ap.add_argument("--rukedra-sizes", default="compact,wide", help="which size points of benchmarks/rukedra_bench.py::SIZES to run")
     ap.add_argument("--rukedra-model-only", action="store_true", help="skip the per-kernel table (a short run for a kernel trace)")
     ap.add_argument("--no-reference-order", action="store_true",
@@ -955,6 +962,11 @@ def main():
         from benchmarks.rukedra_bench import run as rukedra_run
 
         print(json.dumps(rukedra_run(args.layered_dtype, sizes=tuple(args.rukedra_sizes.split(",")), kernels=not args.rukedra_model_only)))
+        return
+    if args.kokuvik:
+        from benchmarks.kokuvik_bench import run as kokuvik_run
+
+        print(json.dumps(kokuvik_run(args.layered_dtype, sizes=tuple(args.kokuvik_sizes.split(",")), kernels=not args.kokuvik_model_only)))
         return
     if args.tusasun:
         from benchmarks.tusasun_bench import run as tusasun_run
