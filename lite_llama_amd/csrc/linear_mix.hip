@@ -375,6 +375,76 @@ __global__ __launch_bounds__(256) void gated_out_norm_block_kernel(void* __restr
   }
 }
 
+// sum over the 16 lanes of a DPP row (every lane of the row active); the result is in every lane of the row
+__device__ __forceinline__ float row16_sum(float v) {
+  float t;
+  t = ll_dpp_f32<0xB1>(v); v += t;   // quad_perm [1,0,3,2]
+  t = ll_dpp_f32<0x4E>(v); v += t;   // quad_perm [2,3,0,1]
+  t = ll_dpp_f32<0x124>(v); v += t;  // row_ror:4
+  t = ll_dpp_f32<0x128>(v); v += t;  // row_ror:8
+  return v;
+}
+
+// The read-out norm of short parts (a head: up to 128 NP channels, a multiple of 8) in 16-byte pieces: one 16-lane row per (token,
+// part), lane r owns the eight channels at 8 (r + 16 j).  Every value is read once; same arithmetic per element as the wave form.
+template <int DT, int NP>
+__global__ __launch_bounds__(256) void gated_out_norm_vec_kernel(void* __restrict__ out, int64_t out_ld, const float* __restrict__ o,
+                                                                 const void* __restrict__ gate, int64_t gate_ld, int gate_kind,
+                                                                 int gate_first, const void* __restrict__ w, int w_len, float eps,
+                                                                 float out_scale, int64_t items, int parts, int ps) {
+  const int64_t item = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  if (item >= items) return;   // (whole 16-lane rows leave; nothing below crosses rows)
+  const int r = threadIdx.x & 15;
+  const int64_t t = item / parts;
+  const int c0 = (int)(item - t * parts) * ps;
+  float v[NP][8], g[NP][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int cc = 8 * (r + 16 * j);
+    const bool in = cc < ps;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      v[j][e] = 0.f;
+      g[j][e] = 1.f;
+    }
+    if (in) {
+      ld8<LL_F32>(o, t * (int64_t)parts * ps + c0 + cc, v[j]);
+      if (gate_kind) {
+        ld8<DT>(gate, t * gate_ld + c0 + cc, g[j]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float s = act_sigmoid<DT>(g[j][e]);
+          g[j][e] = gate_kind == 1 ? g[j][e] * s : s;
+        }
+      }
+      if (gate_first) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[j][e] *= g[j][e];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += v[j][e] * v[j][e];
+  }
+  ss = row16_sum(ss);
+  const float inv = 1.0f / sqrtf(ss / (float)ps + eps);
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int cc = 8 * (r + 16 * j);
+    if (cc < ps) {
+      float wv[8];
+      if (w) ld8<DT>(w, (c0 + cc) % w_len, wv);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        float y = v[j][e] * inv * (w ? wv[e] : 1.0f);
+        if (!gate_first) y *= g[j][e];
+        v[j][e] = y * out_scale;
+      }
+      st8<DT>(out, t * out_ld + c0 + cc, v[j]);
+    }
+  }
+}
+
 // The convolution in 16-byte pieces: a thread owns eight consecutive channels of one token; the taps' weights of those
 // channels are one contiguous run of 8 TAPS values.  Same sums in the same order as the plain form.
 template <int DT, int TAPS>
@@ -596,6 +666,22 @@ extern "C" int ll_gated_out_norm(void* out, int64_t out_ld, const float* o, cons
       out, out_ld, o, gate, gate_ld, gate_kind, gate_first ? 1 : 0, w, (int)(w ? w_len : 1), eps, out_scale, (int)parts, (int)(width / parts))
     LL_BY_DTYPE(dtype, CALL);
 #undef CALL
+    return LL_LAUNCH_CHECK();
+  }
+  const int al = dtype == LL_F32 ? 4 : 8, ps = (int)(width / parts);
+  if (ps % 8 == 0 && ps <= 512 && out_ld % al == 0 && ll_aligned16(out) && ll_aligned16(o) &&
+      (!gate_kind || (gate_ld % al == 0 && ll_aligned16(gate))) && (!w || (w_len % 8 == 0 && ll_aligned16(w)))) {
+    const dim3 vgrid((unsigned)((items + 15) / 16));
+#define CALL_N(DT, NP)                                                                                                           \
+  gated_out_norm_vec_kernel<DT, NP><<<vgrid, 256, 0, (hipStream_t)stream>>>(                                                     \
+      out, out_ld, o, gate, gate_ld, gate_kind, gate_first ? 1 : 0, w, (int)(w ? w_len : 8), eps, out_scale, items, (int)parts, ps)
+#define CALL(DT)                      \
+  if (ps <= 128) CALL_N(DT, 1);       \
+  else if (ps <= 256) CALL_N(DT, 2);  \
+  else CALL_N(DT, 4)
+    LL_BY_DTYPE(dtype, CALL);
+#undef CALL
+#undef CALL_N
     return LL_LAUNCH_CHECK();
   }
 #define CALL(DT)                                                                                                                 \

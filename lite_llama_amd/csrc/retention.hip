@@ -69,6 +69,8 @@ __device__ __forceinline__ float rotated_entry(const void* p, int64_t at, int i,
 // ------------------------------------------------------------------------------------------------------------------------
 // decoded tokens.  Thread (row group g, piece): CV neighbouring state columns, key entries g, g + groups, ..
 // ------------------------------------------------------------------------------------------------------------------------
+constexpr int kRows = 8;   // state rows in flight per thread
+
 template <int DT, int CV>
 __global__ __launch_bounds__(256) void retention_decode_kernel(const RetentionArgs a) {
   extern __shared__ float lds[];
@@ -99,26 +101,37 @@ __global__ __launch_bounds__(256) void retention_decode_kernel(const RetentionAr
         val[e] = ldv<DT>(a.v, t * a.v_ld + (int64_t)head * dv + pc * CV + e);
         acc[e] = 0.f;
       }
-#pragma unroll 8
-      for (int r = g; r < dk; r += groups) {
-        float S[CV];
-        float* sp = st + (int64_t)r * dv + pc * CV;
-        if constexpr (CV == 4) {
-          f32x4 old = {0.f, 0.f, 0.f, 0.f};
-          if (carry) old = *reinterpret_cast<const f32x4*>(sp);
+      // eight rows of the state at a time: all of them are requested before the first is written back
+      for (int r0 = g; r0 < dk; r0 += kRows * groups) {
+        float S[kRows][CV];
 #pragma unroll
-          for (int e = 0; e < 4; ++e) S[e] = old[e];
-        } else {
-          S[0] = carry ? sp[0] : 0.f;
-        }
-        const float kr = sk[r], qr = sq[r];
+        for (int j = 0; j < kRows; ++j) {
+          const int r = r0 + j * groups;
+          const float* sp = st + (int64_t)r * dv + pc * CV;
+          const bool in = carry && r < dk;
+          if constexpr (CV == 4) {
+            f32x4 old = {0.f, 0.f, 0.f, 0.f};
+            if (in) old = *reinterpret_cast<const f32x4*>(sp);
 #pragma unroll
-        for (int e = 0; e < CV; ++e) {
-          S[e] = __builtin_fmaf(dec, S[e], kr * val[e]);
-          acc[e] = __builtin_fmaf(S[e], qr, acc[e]);
+            for (int e = 0; e < 4; ++e) S[j][e] = old[e];
+          } else {
+            S[j][0] = in ? sp[0] : 0.f;
+          }
         }
-        if constexpr (CV == 4) *reinterpret_cast<f32x4*>(sp) = f32x4{S[0], S[1], S[2], S[3]};
-        else sp[0] = S[0];
+#pragma unroll
+        for (int j = 0; j < kRows; ++j) {
+          const int r = r0 + j * groups;
+          if (r >= dk) break;
+          float* sp = st + (int64_t)r * dv + pc * CV;
+          const float kr = sk[r], qr = sq[r];
+#pragma unroll
+          for (int e = 0; e < CV; ++e) {
+            S[j][e] = __builtin_fmaf(dec, S[j][e], kr * val[e]);
+            acc[e] = __builtin_fmaf(S[j][e], qr, acc[e]);
+          }
+          if constexpr (CV == 4) *reinterpret_cast<f32x4*>(sp) = f32x4{S[j][0], S[j][1], S[j][2], S[j][3]};
+          else sp[0] = S[j][0];
+        }
       }
 #pragma unroll
       for (int e = 0; e < CV; ++e) so[g * dv + pc * CV + e] = acc[e];
@@ -332,36 +345,41 @@ __global__ __launch_bounds__(256) void retention_chunk_kernel(const RetentionArg
       for (int j = 0; j < 2; ++j) *reinterpret_cast<f32x4*>(ss + (16 * j + t) * KS + 16 * (wave + 4 * i) + 4 * c) = S[i][j];
     __syncthreads();
     if (base + kC < t1) fetch(base + kC);
-    // scores of keys 16 ct .. against queries 16 tt .. (keys behind every query of the tile: zeros)
-    f32x4 p = {0.f, 0.f, 0.f, 0.f};
-    if (ct <= tt) {
+    // scores of keys 16 ct .. against queries 16 tt .. (keys behind every query of the tile: zeros), and the read-out of the state
+    // in front of the chunk: one query fragment feeds both products
+    f32x4 p = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
+    {
+      const float* qp = sq + (16 * tt + t) * KS + 4 * c;
+      const float* kp = sk + (16 * ct + t) * KS + 4 * c;
+      const float* op = ss + (16 * ct + t) * KS + 4 * c;
+      if (ct <= tt) {
 #pragma unroll
-      for (int s = 0; s < KT; ++s) {
-        const f32x4 ka = *reinterpret_cast<const f32x4*>(sk + (16 * ct + t) * KS + 16 * s + 4 * c);
-        const f32x4 qb = *reinterpret_cast<const f32x4*>(sq + (16 * tt + t) * KS + 16 * s + 4 * c);
+        for (int s = 0; s < KT; ++s) {
+          const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + 16 * s), kf = *reinterpret_cast<const f32x4*>(kp + 16 * s),
+                      sf = *reinterpret_cast<const f32x4*>(op + 16 * s);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) p = mfma4(ka[e], qb[e], p);
-      }
+          for (int e = 0; e < 4; ++e) {
+            p = mfma4(kf[e], qf[e], p);
+            o = mfma4(qf[e], sf[e], o);
+          }
+        }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int gap = 16 * (tt - ct) + t - 4 * c - r;
-        p[r] = gap >= 0 ? p[r] * pw[gap] : 0.f;
+        for (int r = 0; r < 4; ++r) {
+          const int gap = 16 * (tt - ct) + t - 4 * c - r;
+          p[r] = gap >= 0 ? p[r] * pw[gap] : 0.f;
+        }
+      } else {
+#pragma unroll
+        for (int s = 0; s < KT; ++s) {
+          const f32x4 qf = *reinterpret_cast<const f32x4*>(qp + 16 * s), sf = *reinterpret_cast<const f32x4*>(op + 16 * s);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o = mfma4(qf[e], sf[e], o);
+        }
       }
     }
     *reinterpret_cast<f32x4*>(sp + (16 * tt + t) * kPS + 16 * ct + 4 * c) = p;
-    // the state in front of the chunk
-    f32x4 o = {0.f, 0.f, 0.f, 0.f};
-    if (carry || base > t0) {
 #pragma unroll
-      for (int s = 0; s < KT; ++s) {
-        const f32x4 qa = *reinterpret_cast<const f32x4*>(sq + (16 * tt + t) * KS + 16 * s + 4 * c);
-        const f32x4 sb = *reinterpret_cast<const f32x4*>(ss + (16 * ct + t) * KS + 16 * s + 4 * c);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) o = mfma4(qa[e], sb[e], o);
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] *= pw[16 * tt + 4 * c + r + 1];
-    }
+    for (int r = 0; r < 4; ++r) o[r] *= pw[16 * tt + 4 * c + r + 1];
     __syncthreads();   // the scores are there
 #pragma unroll
     for (int s = 0; s < kC / 16; ++s) {
