@@ -189,13 +189,16 @@ __global__ __launch_bounds__(64) void group_select_kernel(const float* __restric
     else extra_scale[t] = sigmoid_exact(z);
   }
   __syncthreads();
-  if constexpr (SCORING == 4) {   // the logits become softmax scores: every lane adds all exponentials in index order
+  if constexpr (SCORING == 4) {   // the logits become softmax scores; every lane adds all exponentials in index order
     float top_z = -INFINITY;
     for (int e = 0; e < experts; ++e) top_z = fmaxf(top_z, score[e]);
-    float total = 0.f;
-    for (int e = 0; e < experts; ++e) total += expf(score[e] - top_z);
     __syncthreads();
-    for (int e = lane; e < experts; e += 64) score[e] = expf(score[e] - top_z) / total;
+    for (int e = lane; e < experts; e += 64) score[e] = expf(score[e] - top_z);
+    __syncthreads();
+    float total = 0.f;
+    for (int e = 0; e < experts; ++e) total += score[e];
+    __syncthreads();
+    for (int e = lane; e < experts; e += 64) score[e] /= total;
     __syncthreads();
   }
   const int per = experts / group_count;

@@ -654,3 +654,24 @@ def test_random_configurations_whole_in_portions_decoded_and_side_by_side(tmp_pa
     runner.check_errors()
     _close(torch.cat(got_a), wa, 5e-5)
     _close(torch.cat(got_b), wb, 5e-5)
+
+
+@pytest.mark.parametrize("seed", range(20, 28))
+def test_random_configurations_in_bfloat16_track_the_oracle_and_their_own_portions(tmp_path, seed):
+    from lite_llama_amd.executor.ragged import RaggedRunner
+    from lite_llama_amd.weights import load_pretrained
+    from oracle import kokuvik as O
+
+    cfg = _random_config(seed)
+    tens = T.tensors(cfg, seed=seed)
+    model = load_pretrained(L.write(tmp_path / "m", cfg, tens), device=DEV, dtype=torch.bfloat16)
+    a = L.prompt(cfg, 150, seed=seed)
+    want = O.forward(a, tens, cfg)
+    runner = RaggedRunner(model, 512, 2, device=DEV)
+    whole = _feed(runner, runner.admit(), a, [150]).float().cpu()
+    parts = _feed(runner, runner.admit(), a, [2, 9, 40, 1, 65, 1]).float().cpu()
+    runner.check_errors()
+    # medians over the tokens: a close call of a router may go the other way
+    err = lambda x, y: (x.to(F64) - y.to(F64)).pow(2).mean(-1).sqrt().median().item()   # noqa: E731
+    assert err(whole, want) < 0.06 * want.std().item()
+    assert err(parts, whole) < 0.04 * want.std().item()
