@@ -297,7 +297,7 @@ def test_window_edge_with_kept_keys_in_prompts_and_in_decoding(dtype, shape, win
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("shape", SHAPES[:3])
 @pytest.mark.parametrize("sink", [-40.0, 2.0, 12.0])
-def test_learned_sink_takes_its_share_and_counts_once(dtype, shape, sink):
+def test_learned_sink_enters_the_denominator_once(dtype, shape, sink):
     """Contexts that span several partitions of the decoded form: a sink counted per partition would show at once; a dominant sink
     leaves nearly nothing, a faint one everything."""
     total = 620
